@@ -1,5 +1,6 @@
 from .base import ConfigError, ModelConfig, read_config_json
 from .mumusun import MumusunConfig
+from .narasun import NarasunConfig
 from .podurax import PoduraxConfig
 from .qwen2 import Qwen2Config
 from .tabatar import TabatarConfig

@@ -206,6 +206,17 @@ class LoopConfig:
         return {"start": self.start, "stop": self.stop, "times": self.times}
 
 
+def run_order_with_passes(loop: Optional[LoopConfig], n_layers: int) -> Tuple[Tuple[int, Optional[int]], ...]:
+    """(layer, pass) in the order the layers run: the looped span ``times`` times in a row, the others once.  ``pass`` is the
+    number of the pass on the first layer of every pass of the loop and None everywhere else."""
+    if loop is None:
+        return tuple((i, None) for i in range(n_layers))
+    out = [(i, None) for i in range(loop.start)]
+    for t in range(loop.times):
+        out += [(i, t if i == loop.start else None) for i in range(loop.start, loop.stop)]
+    return tuple(out + [(i, None) for i in range(loop.stop, n_layers)])
+
+
 @dataclasses.dataclass(frozen=True)
 class TabatarConfig(ModelConfig):
     vocab: int

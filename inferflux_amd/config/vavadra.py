@@ -26,7 +26,7 @@ from typing import Any, ClassVar, Dict, Mapping, Optional, Tuple, Union
 
 from .base import ConfigError, ModelConfig, read_key
 from .mumusun import _read, _section
-from .tabatar import LoopConfig
+from .tabatar import LoopConfig, run_order_with_passes
 
 MIXER_TYPES = ("attention", "delta", "latent_attention")
 MLP_KINDS = ("moe",)
@@ -269,16 +269,8 @@ class VavadraConfig(ModelConfig):
                 L.mlp.validate(f"layers[{i}].mlp.")
 
     def run_order(self) -> Tuple[Tuple[int, Optional[int]], ...]:
-        """(layer, pass) in the order the layers run: the looped span ``times`` times in a row, the others once.  ``pass`` is
-        the number of the pass on the first layer of every pass of the loop and None everywhere else."""
-        n = len(self.layers)
-        if self.loop is None:
-            return tuple((i, None) for i in range(n))
-        lp = self.loop
-        out = [(i, None) for i in range(lp.start)]
-        for t in range(lp.times):
-            out += [(i, t if i == lp.start else None) for i in range(lp.start, lp.stop)]
-        return tuple(out + [(i, None) for i in range(lp.stop, n)])
+        """(layer, pass) in the order the layers run (see ``run_order_with_passes``)."""
+        return run_order_with_passes(self.loop, len(self.layers))
 
     def open_sizes(self) -> Tuple[str, ...]:
         return tuple(f"layers[{i}].mixer.conv" for i, L in enumerate(self.layers) if L.type == "delta" and L.mixer.conv is None)

@@ -46,7 +46,7 @@ extern "C" int ifx_embedding(const int* ids, const void* table, int table_dtype,
 // product that reads ``rows`` multiplies its sums by rsqrt(sum of the pieces / H + eps) (RowScale in gemm_bf16.hip).
 template <typename T>
 __global__ __launch_bounds__(256) void embedding_norm_kernel(const int* __restrict__ ids, const T* __restrict__ table,
-                                                            const bf16_t* __restrict__ norm_w, float* __restrict__ out,
+                                                            const void* __restrict__ norm_w, int norm_dtype, float* __restrict__ out,
                                                             bf16_t* __restrict__ rows, float* __restrict__ pieces,
                                                             int n_rows, int H, float scale) {
   __shared__ float red[16];
@@ -57,7 +57,7 @@ __global__ __launch_bounds__(256) void embedding_norm_kernel(const int* __restri
     for (int i = i0 + threadIdx.x; i < i1; i += blockDim.x) {
       const float x = to_f(src[i]) * scale;
       out[(size_t)t * H + i] = x;
-      rows[(size_t)t * H + i] = (bf16_t)(x * to_f(norm_w[i]));
+      rows[(size_t)t * H + i] = (bf16_t)(x * load_dyn(norm_w, norm_dtype, i));
       ss += x * x;
     }
   }
@@ -65,7 +65,7 @@ __global__ __launch_bounds__(256) void embedding_norm_kernel(const int* __restri
   if (threadIdx.x == 0) pieces[run * 16 + t] = ss;
 }
 
-extern "C" int ifx_embedding_norm(const int* ids, const void* table, int table_dtype, const void* norm_w, float* out,
+extern "C" int ifx_embedding_norm(const int* ids, const void* table, int table_dtype, const void* norm_w, int norm_dtype, float* out,
                                   void* rows, float* pieces, int T, int H, float scale, void* stream) {
   IFX_REQUIRE(T >= 0 && T <= 16 && H > 0, "embedding_norm: T=%d must be at most 16 (H=%d)", T, H);
   IFX_REQUIRE(norm_w && out && rows && pieces, "embedding_norm: needs the norm's weight and three outputs");
@@ -73,9 +73,9 @@ extern "C" int ifx_embedding_norm(const int* ids, const void* table, int table_d
   hipStream_t s = (hipStream_t)stream;
   const dim3 grid(16, (H + 4095) / 4096);
   if (table_dtype == DT_F32)
-    hipLaunchKernelGGL(embedding_norm_kernel<float>, grid, dim3(256), 0, s, ids, (const float*)table, (const bf16_t*)norm_w, out, (bf16_t*)rows, pieces, T, H, scale);
+    hipLaunchKernelGGL(embedding_norm_kernel<float>, grid, dim3(256), 0, s, ids, (const float*)table, norm_w, norm_dtype, out, (bf16_t*)rows, pieces, T, H, scale);
   else if (table_dtype == DT_BF16)
-    hipLaunchKernelGGL(embedding_norm_kernel<bf16_t>, grid, dim3(256), 0, s, ids, (const bf16_t*)table, (const bf16_t*)norm_w, out, (bf16_t*)rows, pieces, T, H, scale);
+    hipLaunchKernelGGL(embedding_norm_kernel<bf16_t>, grid, dim3(256), 0, s, ids, (const bf16_t*)table, norm_w, norm_dtype, out, (bf16_t*)rows, pieces, T, H, scale);
   else
     IFX_FAIL("embedding_norm: unknown dtype %d", table_dtype);
   IFX_LAUNCH_CHECK();
@@ -391,6 +391,7 @@ struct RopeArgs {
   int pre_norm_dtype;
   float pre_norm_eps;
   int extra_cols;        // further columns at the end of a row that this kernel does not read (another kernel's)
+  const float* q_mult;   // [T]: a factor on every query of row t, applied in float before the rounding (null: none)
 };
 
 template <typename T>
@@ -473,7 +474,7 @@ __global__ __launch_bounds__(64) void rope_append_kernel(RopeArgs a) {
         y1 = x0 * sn + x1 * cs;
       }
     };
-    float inv = 1.f;
+    float inv = is_q && a.q_mult ? a.q_mult[t] : 1.f;
     if (a.unit_norm) {       // the head's sum of squares first (the block is one wave); the values are formed again below
       float ss = 0.f;
       for (int p = threadIdx.x; p < half; p += blockDim.x) {
@@ -482,7 +483,7 @@ __global__ __launch_bounds__(64) void rope_append_kernel(RopeArgs a) {
         pair(p, i0, i1, y0, y1);
         ss += y0 * y0 + y1 * y1;
       }
-      inv = rsqrtf(wave_sum(ss) / (float)d + a.norm_eps);
+      inv *= rsqrtf(wave_sum(ss) / (float)d + a.norm_eps);
     }
     for (int p = threadIdx.x; p < half; p += blockDim.x) {
       int i0, i1;
@@ -652,13 +653,13 @@ __global__ __launch_bounds__(256) void rope_append_vec_x_kernel(RopeArgs a, int 
         f1[e] = u * sn[e] + w * cs[e];
       }
     }
-    float inv = 1.f;
+    float inv = head < a.nH && a.q_mult ? a.q_mult[t] : 1.f;
     if (a.unit_norm) {
       float ss = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) ss += f0[e] * f0[e] + f1[e] * f1[e];
       for (int o = per_head / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, WAVE);     // the head's threads are neighbours
-      inv = rsqrtf(ss / (float)d + a.norm_eps);
+      inv *= rsqrtf(ss / (float)d + a.norm_eps);
     }
     if (head < a.nH && a.gate_cols && j == 0) {
       const int gc = q_width + kv_width + v_width + head;
@@ -732,7 +733,7 @@ extern "C" int ifx_rope_append(const void* qkv, int dtype, const void* bias, int
                                int nKV, int d, int page_size, void* q_out, void* k_cache, void* v_cache, int n_slices,
                                long long slice_stride, int dv, int gate_cols, float* gate_out, int unit_norm, float norm_eps,
                                const void* v_first, float v_mix, void* v_out, const void* q_norm_w, const void* k_norm_w,
-                               int pre_norm_dtype, float pre_norm_eps, int extra_cols, void* stream) {
+                               int pre_norm_dtype, float pre_norm_eps, int extra_cols, const float* q_mult, void* stream) {
   IFX_REQUIRE((q_norm_w != nullptr) == (k_norm_w != nullptr) && extra_cols >= 0, "rope_append: norms for q and k come together");
   IFX_REQUIRE(n_slices >= 1 && (n_slices == 1 || slice_stride > 0), "rope_append: %d slices, %lld apart", n_slices, slice_stride);
   IFX_REQUIRE(T >= 0 && nH > 0 && nKV >= 0 && d > 0 && d % 2 == 0 && dv > 0, "rope_append: bad sizes T=%d nH=%d nKV=%d d=%d dv=%d", T, nH, nKV, d, dv);
@@ -746,8 +747,8 @@ extern "C" int ifx_rope_append(const void* qkv, int dtype, const void* bias, int
   IFX_REQUIRE(!(v_first || v_out) || nKV > 0, "rope_append: values to mix or to hand on, but no kv heads");
   RopeArgs a{qkv, n_slices, (size_t)slice_stride, bias, bias_dtype, slots, cs, sn, rope_style, rotary_dim, nH, nKV, d, page_size,
              q_out, k_cache, v_cache, dv, gate_cols, gate_out, unit_norm, norm_eps, v_first, v_mix, v_out,
-             q_norm_w, k_norm_w, pre_norm_dtype, pre_norm_eps, extra_cols};
-  const bool extras = gate_cols || unit_norm || v_first || v_out || q_norm_w || extra_cols;
+             q_norm_w, k_norm_w, pre_norm_dtype, pre_norm_eps, extra_cols, q_mult};
+  const bool extras = gate_cols || unit_norm || v_first || v_out || q_norm_w || extra_cols || q_mult;
   hipStream_t s = (hipStream_t)stream;
   // (a few tokens are quicker with one small block per token and head: nothing waits on a loop over tokens)
   if (!extras && dv == d && T >= 128 && n_slices == 1 && dtype == DT_BF16 && rope_style == 1 && rotary_dim == d && d % 16 == 0 && (!bias || bias_dtype == DT_BF16) &&
@@ -826,3 +827,17 @@ extern "C" int ifx_swiglu(const void* gu, void* out, int dtype, int T, int I, in
   IFX_LAUNCH_CHECK();
 }
 
+
+// ---------------------------------------------------------------------------------------
+// out[t] = 1 + coef * ln(floor((positions[t] + 1) / every) + 1)
+__global__ __launch_bounds__(256) void query_temperature_kernel(const int* __restrict__ positions, float* __restrict__ out, int T, float coef, int every) {
+  const int t = blockIdx.x * 256 + threadIdx.x;
+  if (t < T) out[t] = fmaf(coef, logf((float)((positions[t] + 1) / every + 1)), 1.0f);
+}
+
+extern "C" int ifx_query_temperature(const int* positions, float* out, int T, float coef, int every, void* stream) {
+  IFX_REQUIRE(T >= 0 && every > 0, "query_temperature: T=%d every=%d", T, every);
+  if (T == 0) return 0;
+  hipLaunchKernelGGL(query_temperature_kernel, dim3((T + 255) / 256), dim3(256), 0, (hipStream_t)stream, positions, out, T, coef, every);
+  IFX_LAUNCH_CHECK();
+}

@@ -40,11 +40,16 @@ __device__ __forceinline__ bf16x8 zero8() {
 // written beside it: rows[m, n] = bf16(stream[m, n] * norm_w[n]) and pieces[n / 16][m] (see RowScale).
 struct StreamOut {
   float* stream;
-  const bf16_t* norm_w;
+  const void* norm_w;      // bfloat16, or float (a weight formed at load: norm_f32)
+  int norm_f32;
   bf16_t* rows;
   float* pieces;
   float mult;      // the product is multiplied by this before it is added (a model's factor on every sub-block's output)
 };
+
+// A product whose weight's row tiles come in blocks that read inputs of their own: row tile t meets x + min(t / tiles, n - 1) * M * K
+// (x holds n inputs [M, K] end to end; tiles 0: one input for all).
+struct XBlocks { int tiles, n; };
 
 // Sum over the four lanes col, col + 16, col + 32, col + 48, the same in all four.
 __device__ __forceinline__ float sum_over_groups(float v) {
@@ -149,7 +154,7 @@ typedef __attribute__((__vector_size__(2 * sizeof(float)))) float floatx2;
 template <int MT, int NT, int U, typename TO, int EPI, bool TILED>
 __global__ void skinny_gemm_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ W, TO* __restrict__ out,
                                    int M, int N, int K, int k_tiles, const int* __restrict__ order, RowScale scale,
-                                   StreamOut so, int tile_rows) {
+                                   StreamOut so, int tile_rows, XBlocks xb) {
   extern __shared__ float red[];  // [(waves - 1)][NT * MT][64 lanes][4]
   const int lane = threadIdx.x % WAVE, col = lane & 15, g = lane >> 4;
   const int first_tile = blockIdx.x * NT, n_tiles = (N + tile_rows - 1) / tile_rows;
@@ -160,7 +165,7 @@ __global__ void skinny_gemm_kernel(const bf16_t* __restrict__ x, const bf16_t* _
   // pair is held or not as a whole, and a pair's first column is even.
   // EPI 2: what the epilogue reads is asked for before the stream of weights, not after it
   floatx2 was[NT][2];
-  bf16x2 nw[NT][2];
+  floatx2 nw[NT][2];
   if (EPI == 2 && first_wave) {
 #pragma unroll
     for (int nt = 0; nt < NT; ++nt)
@@ -169,10 +174,16 @@ __global__ void skinny_gemm_kernel(const bf16_t* __restrict__ x, const bf16_t* _
         const int n = tile_rows * (first_tile + nt) + 4 * g + 2 * q;
         const bool ok = 4 * g + 2 * q < tile_rows && n < N && col < M;
         was[nt][q] = ok ? *(const floatx2*)(so.stream + (size_t)col * N + n) : floatx2{0.f, 0.f};
-        if (ok) nw[nt][q] = *(const bf16x2*)(so.norm_w + n);
+        nw[nt][q] = floatx2{0.f, 0.f};
+        if (ok && so.norm_f32) nw[nt][q] = *(const floatx2*)((const float*)so.norm_w + n);
+        else if (ok) {
+          const bf16x2 w2 = *(const bf16x2*)((const bf16_t*)so.norm_w + n);
+          nw[nt][q] = floatx2{(float)w2[0], (float)w2[1]};
+        }
       }
   }
   floatx4 acc[NT][MT];
+  if (xb.tiles > 0) x += (size_t)min(first_tile / xb.tiles, xb.n - 1) * M * K;
   if (!skinny_accumulate<MT, NT, U, TILED>(x, W, M, N, K, k_tiles, first_tile, acc, red, tile_rows)) return;
   // acc[nt][mt][r] = out[m = 16 mt + col][n = tile_rows (row tile of the weight) + 4 g + r], for 4 g + r < tile_rows
   if (EPI == 2) {
@@ -189,7 +200,7 @@ __global__ void skinny_gemm_kernel(const bf16_t* __restrict__ x, const bf16_t* _
 #pragma unroll
           for (int r = 0; r < 2; ++r) {
             v[r] = was[nt][q][r] + acc[nt][0][2 * q + r] * rs * so.mult;
-            y[r] = (__bf16)(v[r] * (float)nw[nt][q][r]);
+            y[r] = (__bf16)(v[r] * nw[nt][q][r]);
             sq += v[r] * v[r];
           }
           *(floatx2*)(so.stream + (size_t)col * N + n) = v;
@@ -306,13 +317,13 @@ __global__ void qkv_rope_kernel(const bf16_t* __restrict__ x, const bf16_t* __re
 
 template <int MT, int NT, int U, bool TILED>
 static int launch(const void* x, const void* W, void* out, int out_dtype, int M, int N, int K, int k_tiles, int waves, int epi,
-                  const int* order, const RowScale& scale, const StreamOut& so, int tile_rows, hipStream_t s) {
+                  const int* order, const RowScale& scale, const StreamOut& so, int tile_rows, XBlocks xb, hipStream_t s) {
   const int groups = ((N + tile_rows - 1) / tile_rows + NT - 1) / NT;
   const size_t lds = (size_t)(waves - 1) * NT * MT * WAVE * 4 * sizeof(float);
   IFX_REQUIRE(lds <= 64 * 1024, "skinny_gemm: %d waves of %dx%d tiles need %zu bytes of LDS", waves, NT, MT, lds);
 #define GO(TO_, EPI_)                                                                                              \
   hipLaunchKernelGGL((skinny_gemm_kernel<MT, NT, U, TO_, EPI_, TILED>), dim3(groups), dim3(waves * WAVE), lds, s,  \
-                     (const bf16_t*)x, (const bf16_t*)W, (TO_*)out, M, N, K, k_tiles, order, scale, so, tile_rows)
+                     (const bf16_t*)x, (const bf16_t*)W, (TO_*)out, M, N, K, k_tiles, order, scale, so, tile_rows, xb)
   if (epi == 2) {
     if constexpr (MT == 1) GO(float, 2);
     else IFX_FAIL("skinny_gemm: the stream epilogue takes at most 16 rows");
@@ -400,14 +411,16 @@ extern "C" int ifx_qkv_rope(const void* x, const void* Wt, int M, int K, const v
 // epi 1: gate/up rows interleaved in W, out = silu(gate) * up, [M, N / 2]; epi 3: the same with the tanh form of gelu.
 // epi 2: the product is added to ``stream`` [M, N] (float, in place), rows_out [M, N] = bf16(stream * norm_w) and
 //        pieces_out [ceil(N / 16)][16] = sums of squares of the stream in runs of 16, for the norm that follows
-//        (M <= 16, N a multiple of 4, norm_w bfloat16 [N]); ``out`` is not used.
+//        (M <= 16, N a multiple of 4, norm_w [N] bfloat16, or float with norm_f32); ``out`` is not used.
+// block_tiles, n_blocks: row tiles in blocks that read inputs of their own (see XBlocks; block_tiles 0: one input).
 // tiled 1 or 16: W is the tiled form written by ifx_tile_weights, with the row-tile order it was given (or null);
 //        8 to 14 (even): that form with so many rows to a tile (no order).
 // scale_pieces [n_scale_pieces][16] (or null), scale_width, scale_eps: a factor per row of x (M <= 16), see RowScale.
 extern "C" int ifx_skinny_gemm(const void* x, const void* W, void* out, int out_dtype, int M, int N, int K, int nt,
                                int waves, int unroll, int epi, int tiled, const int* order, const float* scale_pieces,
                                int n_scale_pieces, float scale_width, float scale_eps, float* stream_io,
-                               const void* norm_w, void* rows_out, float* pieces_out, float stream_mult, void* stream) {
+                               const void* norm_w, int norm_f32, void* rows_out, float* pieces_out, float stream_mult, int block_tiles,
+                               int n_blocks, void* stream) {
   IFX_REQUIRE(tiled == 0 || tiled == 1 || (tiled >= 8 && tiled <= 16 && tiled % 2 == 0), "skinny_gemm: tiled=%d (0, 1, or 8 to 16 rows to a tile)", tiled);
   const int tile_rows = tiled >= 8 ? tiled : 16;
   IFX_REQUIRE((tiled && tile_rows == 16) || !order, "skinny_gemm: a tile order goes with a tiled copy of 16-row tiles");
@@ -465,11 +478,14 @@ extern "C" int ifx_skinny_gemm(const void* x, const void* W, void* out, int out_
   hipStream_t s = (hipStream_t)stream;
   const int k_tiles = ifx_tiled_cols(K) / 32;
   const RowScale scale{scale_pieces, n_scale_pieces, scale_width, scale_eps};
-  const StreamOut so{stream_io, (const bf16_t*)norm_w, (bf16_t*)rows_out, pieces_out, stream_mult};
+  const StreamOut so{stream_io, norm_w, norm_f32, (bf16_t*)rows_out, pieces_out, stream_mult};
+  IFX_REQUIRE(block_tiles == 0 || (block_tiles > 0 && n_blocks > 0 && epi == 0 && !order && (block_tiles % 2 == 0 || nt == 1)),
+              "skinny_gemm: blocks of %d tiles with inputs of their own go with the plain epilogue (and an even number of tiles, or one a wave)", block_tiles);
+  const XBlocks xb{block_tiles, n_blocks};
 #define CASE(MT_, NT_, U_)                                                                                             \
   if (mt == MT_ && nt == NT_ && unroll == U_)                                                                          \
-    return tiled ? launch<MT_, NT_, U_, true>(x, W, out, out_dtype, M, N, K, k_tiles, waves, epi, order, scale, so, tile_rows, s)  \
-                 : launch<MT_, NT_, U_, false>(x, W, out, out_dtype, M, N, K, k_tiles, waves, epi, order, scale, so, 16, s)
+    return tiled ? launch<MT_, NT_, U_, true>(x, W, out, out_dtype, M, N, K, k_tiles, waves, epi, order, scale, so, tile_rows, xb, s)  \
+                 : launch<MT_, NT_, U_, false>(x, W, out, out_dtype, M, N, K, k_tiles, waves, epi, order, scale, so, 16, xb, s)
   // (the combinations left out need more than the 128 registers a workgroup of 16 waves leaves a lane)
   CASE(1, 1, 4); CASE(1, 2, 4); CASE(1, 1, 2); CASE(1, 2, 2);
   CASE(2, 1, 4); CASE(2, 2, 2); CASE(2, 1, 2);

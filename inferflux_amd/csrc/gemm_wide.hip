@@ -70,6 +70,10 @@ __device__ __forceinline__ void store2(bf16_t* p, float a, float b) {
   *(bf16x2*)p = w;
 }
 
+// A product whose weight's row tiles come in blocks that read inputs of their own: row tile t meets x + min(t / tiles, n - 1) * M * K
+// (x holds n inputs [M, K] end to end, a workgroup's tiles lie within one block; tiles 0: one input for all).
+struct XBlocks { int tiles, n; };
+
 // EPI 0: out[m, n] = sum.  EPI 1: the rows of W alternate gate, up, ...: out[m, n / 2] = silu(gate) * up.
 // ``order``: tile t of the copy holds the weight's rows 16 order[t] ...; null: in order.
 // ``MINW``: the fewest waves a workgroup of this form may have (each thread then copies more pieces of x to LDS and
@@ -81,7 +85,7 @@ template <int MT, typename TO, int EPI, int MINW>
 __global__ __launch_bounds__((16 * MT > MANY_ROWS || MINW < MIN_WAVES ? MIN_WAVES : MAX_WAVES) * WAVE) void wide_gemm_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ Wt,
                                                                      TO* __restrict__ out, float* __restrict__ part, int M,
                                                                      int N, int K, int k_tiles, int rounds_per_slice,
-                                                                     const int* __restrict__ order, int tile_rows, RowScale scale) {
+                                                                     const int* __restrict__ order, int tile_rows, RowScale scale, XBlocks xb) {
   constexpr int R = MT * 16;                                  // rows of x in LDS
   constexpr int X_PIECES = R * WK_PIECES;                     // 16-byte pieces of a round's x
   constexpr int X_PER_THREAD = (X_PIECES + MINW * WAVE - 1) / (MINW * WAVE);
@@ -94,6 +98,7 @@ __global__ __launch_bounds__((16 * MT > MANY_ROWS || MINW < MIN_WAVES ? MIN_WAVE
   if (scaled) row_sums_ask(scale, tid, threads, pieces_asked);
   const int tile = blockIdx.x * waves + wid, n_tiles = (N + tile_rows - 1) / tile_rows;
   const int n_rounds = (K + WK - 1) / WK;
+  if (xb.tiles > 0) x += (size_t)min((int)(blockIdx.x * waves) / xb.tiles, xb.n - 1) * M * K;
   const int r_begin = blockIdx.y * rounds_per_slice, n = min(n_rounds, r_begin + rounds_per_slice) - r_begin;
   // a wave whose tile lies past N reads the last tile again and stores nothing
   // (a tile of the copy holds tile_rows rows, 64 tile_rows bytes per k-tile: see gemm_bf16.hip; the lanes of the other rows hold zeros)
@@ -285,13 +290,13 @@ extern "C" int ifx_wide_gemm_plan(int rows, int N, int K, int waves, int slices,
 
 template <int MT>
 static int launch_wide(const void* x, const void* Wt, void* out, int out_dtype, float* part, int M, int N, int K, int waves,
-                       int slices, int rps, int epi, const int* order, bool add_slices, int tile_rows, RowScale scale, hipStream_t s) {
+                       int slices, int rps, int epi, const int* order, bool add_slices, int tile_rows, RowScale scale, XBlocks xb, hipStream_t s) {
   const int n_tiles = (N + tile_rows - 1) / tile_rows;
   const dim3 grid((n_tiles + waves - 1) / waves, slices);
   const int k_tiles = (K + 63) / 64 * 2;
 #define GO(TO_, EPI_, MINW_)                                                                                       \
   hipLaunchKernelGGL((wide_gemm_kernel<MT, TO_, EPI_, MINW_>), grid, dim3(waves * WAVE), 0, s, (const bf16_t*)x,   \
-                     (const bf16_t*)Wt, (TO_*)out, part, M, N, K, k_tiles, rps, order, tile_rows, scale)
+                     (const bf16_t*)Wt, (TO_*)out, part, M, N, K, k_tiles, rps, order, tile_rows, scale, xb)
 #define GO_ALL(MINW_)                                    \
   if (out_dtype == DT_BF16 && epi == 0) GO(bf16_t, 0, MINW_); \
   else if (out_dtype == DT_BF16 && epi == 3) GO(bf16_t, 3, MINW_); \
@@ -324,9 +329,14 @@ static int launch_wide(const void* x, const void* Wt, void* out, int out_dtype, 
 // ``out`` null with more than one slice: the partial sums are left in ``part`` for a kernel that adds them itself
 // (ifx_add_rmsnorm, ifx_rope_append).
 // scale_pieces [n_scale_pieces][16] (or null), scale_width, scale_eps: a factor per row of x (M <= 16), see RowScale.
+// block_tiles, n_blocks: row tiles in blocks that read inputs of their own (see XBlocks; block_tiles 0: one input).
 extern "C" int ifx_wide_gemm(const void* x, const void* Wt, void* out, int out_dtype, float* part, int M, int N, int K,
                              int waves, int slices, int epi, const int* order, int tile_rows, const float* scale_pieces,
-                             int n_scale_pieces, float scale_width, float scale_eps, void* stream) {
+                             int n_scale_pieces, float scale_width, float scale_eps, int block_tiles, int n_blocks, void* stream) {
+  IFX_REQUIRE(block_tiles == 0 || (block_tiles > 0 && n_blocks > 0 && epi == 0 && !order && block_tiles % waves == 0),
+              "wide_gemm: blocks of %d tiles with inputs of their own go with the plain epilogue and workgroups that lie within a block (%d waves)",
+              block_tiles, waves);
+  const XBlocks xb{block_tiles, n_blocks};
   IFX_REQUIRE(out || slices > 1, "wide_gemm: no output");
   IFX_REQUIRE(tile_rows >= 8 && tile_rows <= 16 && tile_rows % 2 == 0 && (tile_rows == 16 || !order),
               "wide_gemm: %d rows to a tile (8 to 16, even; a tile order goes with 16)", tile_rows);
@@ -348,13 +358,13 @@ extern "C" int ifx_wide_gemm(const void* x, const void* Wt, void* out, int out_d
   IFX_REQUIRE((n_rounds + rps - 1) / rps == slices, "wide_gemm: %d rounds do not cut into %d slices (ask ifx_wide_gemm_plan)", n_rounds, slices);
   hipStream_t s = (hipStream_t)stream;
   switch ((M + 15) / 16) {
-    case 1: return launch_wide<1>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    case 2: return launch_wide<2>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    case 3: return launch_wide<3>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    case 4: return launch_wide<4>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    case 5: return launch_wide<5>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    case 6: return launch_wide<6>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    case 7: return launch_wide<7>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
-    default: return launch_wide<8>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, s);
+    case 1: return launch_wide<1>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    case 2: return launch_wide<2>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    case 3: return launch_wide<3>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    case 4: return launch_wide<4>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    case 5: return launch_wide<5>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    case 6: return launch_wide<6>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    case 7: return launch_wide<7>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
+    default: return launch_wide<8>(x, Wt, out, out_dtype, part, M, N, K, waves, slices, rps, epi, order, out != nullptr, tile_rows, scale, xb, s);
   }
 }

@@ -1,4 +1,5 @@
-// Gated linear attention: a recurrence per head whose state is a matrix and whose decay is a vector per token.
+// Linear recurrences per head whose state is a matrix and whose decay is a vector per token: gated linear attention, and
+// (compiled with TIME_MIX) time mixing with a bonus for the current token.
 //
 // For a request's tokens t = 0, 1, ..., per head, with keys and queries of d channels and values of dv:
 //   alpha_t[i] = sigmoid(z_t[i] + b[i]) ^ (1 / tau) = exp(-softplus(-(z_t[i] + b[i])) / tau)
@@ -6,8 +7,15 @@
 //   o_t[j]     = sum_i S_t[i, j] q_t[i] * q_scale
 //   y_t[j]     = o_t[j] / sqrt(mean_j o_t[j]^2 + eps) * w[j] * silu(g_t[j])
 //
+// Time mixing (keys, queries r and values of d):
+//   w_t[i]     = exp(-exp(z_t[i] + b[i]))
+//   o_t[j]     = sum_i (S_(t-1)[i, j] + u[i] k_t[i] v_t[j]) r_t[i]          (the read-out sees the token's own write only through u)
+//   S_t[i, j]  = w_t[i] S_(t-1)[i, j] + k_t[i] v_t[j]
+//   y_t[j]     = o_t[j] / sqrt(mean_j o_t[j]^2 + eps) * w_norm[head, j] * silu(g_t[j])
+// The bonus' part of o_t is v_t[j] times one number per token, sum_i u[i] k_t[i] r_t[i], which a wave per token forms.
+//
 // Rows are a step's flattened rows (requests end to end, a request's rows in position order).  q, k, v and g are columns
-// of one projected row (the activation type, ld apart); z is float (the decay's second product, without its bias).
+// of projected rows (ld apart); z is float (the decay's second product, without its bias).
 // Decays, their logarithms, S, o, the norm and the gate are float whatever the activation type.
 //
 // A request's S lives in its state slot, one float32 row per slot laid out [head][j][PARTS * DP]: a column j of S as
@@ -27,16 +35,21 @@
 
 IFX_DEFINE_LAST_ERROR()
 
+#ifndef TIME_MIX
+#define TIME_MIX 0
+#endif
+
 #define STAGE 8
 
 struct GlaArgs {
-  const void* rows;        // [T, ld] of the activation type
-  int ld, q_col, k_col, v_col, g_col;
+  const void* q; const void* k; const void* v; const void* g;      // the head-0 columns of row 0; rows ld elements apart
+  int ld;
   const float* z;          // [T, H * d]
   const float* z_bias;     // [H * d] or null
   float inv_tau, q_scale, eps;
-  const void* norm_w;      // [dv]
+  const void* norm_w;      // [dv], or with TIME_MIX [H * dv]
   int norm_dtype;
+  const float* bonus;      // TIME_MIX: u [H * d]
   float* state;            // [slots, state_stride]; S at state_offset of a row
   size_t state_stride, state_offset;
   const int* q_start;      // [R]
@@ -59,7 +72,7 @@ __device__ __forceinline__ float log_sigmoid(float x) {      // -softplus(-x), w
 // (a thread's registers hold DP numbers of S: the more of them, the fewer threads a workgroup may have)
 #define GLA_MAX_THREADS(DP) ((DP) <= 32 ? 1024 : ((DP) <= 64 ? 512 : 256))
 
-template <typename T, int DP, int MODE, int COLS>
+template <typename T, typename TO, int DP, int MODE, int COLS>
 __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
   extern __shared__ float lds[];
   const int d = a.d, dv = a.dv, parts = a.parts, H = a.H;
@@ -68,6 +81,7 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
   float* la = lk + STAGE * d;            // [STAGE][d]
   float* lo = la + STAGE * d;            // [STAGE][dv]
   float* lg = lo + STAGE * dv;           // [STAGE][d]: the decays' logarithms (MODE 1 sums them per channel)
+  __shared__ float lb[STAGE];            // TIME_MIX: sum_i u[i] k[i] q[i] of a token
   const int unit = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
   int t0, n;
   size_t s_at;                            // where this head's S lies
@@ -99,7 +113,7 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
       for (int i = 0; i < DP; ++i) S[c][i] = 0.f;
     }
   }
-  const T* rows = (const T*)a.rows;
+  const T* rq = (const T*)a.q; const T* rk = (const T*)a.k; const T* rv = (const T*)a.v; const T* rg = (const T*)a.g;
   const int wid = tid / WAVE, lane = tid % WAVE, nw = (blockDim.x + WAVE - 1) / WAVE;
   float loga_sum = 0.f;
   for (int s0 = 0; s0 < n; s0 += STAGE) {
@@ -109,9 +123,9 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
       const int tt = it / d, ch = it - tt * d;
       const size_t t = (size_t)(t0 + s0 + tt);
       const float zq = a.z[t * (size_t)(H * d) + head * d + ch] + (a.z_bias ? a.z_bias[head * d + ch] : 0.f);
-      const float kq = to_f(rows[t * a.ld + a.k_col + head * d + ch]);
-      const float qq = MODE == 1 ? 0.f : to_f(rows[t * a.ld + a.q_col + head * d + ch]);
-      const float la_t = log_sigmoid(zq) * a.inv_tau;
+      const float kq = to_f(rk[t * a.ld + head * d + ch]);
+      const float qq = MODE == 1 ? 0.f : to_f(rq[t * a.ld + head * d + ch]);
+      const float la_t = TIME_MIX ? -expf(zq) : log_sigmoid(zq) * a.inv_tau;
       if (MODE == 1) lg[it] = la_t;
       la[it] = expf(la_t);
       lk[it] = kq;
@@ -122,10 +136,19 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
     for (int c = 0; c < COLS; ++c)
 #pragma unroll
       for (int tt = 0; tt < STAGE; ++tt)
-        vv[c][tt] = (j0 + c < dv && tt < ns) ? to_f(rows[(size_t)(t0 + s0 + tt) * a.ld + a.v_col + head * dv + j0 + c]) : 0.f;
+        vv[c][tt] = (j0 + c < dv && tt < ns) ? to_f(rv[(size_t)(t0 + s0 + tt) * a.ld + head * dv + j0 + c]) : 0.f;
     __syncthreads();
     if (MODE == 1 && tid < d)
       for (int tt = 0; tt < ns; ++tt) loga_sum += lg[tt * d + tid];
+    if (TIME_MIX && MODE != 1) {
+      for (int tt = wid; tt < ns; tt += nw) {
+        float b = 0.f;
+        for (int c = lane; c < d; c += WAVE) b = fmaf(a.bonus[head * d + c] * lk[tt * d + c], lq[tt * d + c], b);
+        b = wave_sum(b);
+        if (lane == 0) lb[tt] = b;
+      }
+      __syncthreads();
+    }
     for (int tt = 0; tt < ns; ++tt) {
       const float* aa = la + tt * d + p * DP;
       const float* kk = lk + tt * d + p * DP;
@@ -139,8 +162,9 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
           const float al = aa[i], kv = kk[i], qq = MODE != 1 ? qv[i] : 0.f;
 #pragma unroll
           for (int c = 0; c < COLS; ++c) {
+            if (TIME_MIX && MODE != 1) acc[c] = fmaf(S[c][i], qq, acc[c]);        // (the read-out comes before the write)
             S[c][i] = fmaf(al, S[c][i], kv * vv[c][tt]);
-            if (MODE != 1) acc[c] = fmaf(S[c][i], qq, acc[c]);
+            if (!TIME_MIX && MODE != 1) acc[c] = fmaf(S[c][i], qq, acc[c]);
           }
         }
       }
@@ -149,6 +173,7 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
         for (int c = 0; c < COLS; ++c) {
           float r = acc[c];
           for (int o = 1; o < parts; o <<= 1) r += __shfl_xor(r, o, WAVE);
+          if (TIME_MIX) r = fmaf(lb[tt], vv[c][tt], r);
           if (j0 + c < dv && p == 0) lo[tt * dv + j0 + c] = r;
         }
       }
@@ -162,9 +187,9 @@ __global__ __launch_bounds__(GLA_MAX_THREADS(DP)) void gla_kernel(GlaArgs a) {
         for (int c = lane; c < dv; c += WAVE) ss = fmaf(lo[tt * dv + c], lo[tt * dv + c], ss);
         const float inv = rsqrtf(wave_sum(ss) / (float)dv + a.eps);
         for (int c = lane; c < dv; c += WAVE) {
-          const float g = to_f(rows[t * a.ld + a.g_col + head * dv + c]);
-          ((T*)a.out)[t * (size_t)(H * dv) + head * dv + c] =
-              from_f<T>(lo[tt * dv + c] * inv * load_dyn(a.norm_w, a.norm_dtype, c) * act_silu(g));
+          const float g = to_f(rg[t * a.ld + head * dv + c]);
+          ((TO*)a.out)[t * (size_t)(H * dv) + head * dv + c] =
+              from_f<TO>(lo[tt * dv + c] * inv * load_dyn(a.norm_w, a.norm_dtype, TIME_MIX ? head * dv + c : c) * act_silu(g));
         }
       }
     }
@@ -212,20 +237,20 @@ __global__ __launch_bounds__(256) void gla_combine_kernel(CombineArgs a) {
   *slot = S;
 }
 
-template <typename T, int DP, int MODE, int COLS>
+template <typename T, typename TO, int DP, int MODE, int COLS>
 static void launch_gla_mode(const GlaArgs& a, int units, int threads, size_t lds, hipStream_t s) {
-  hipLaunchKernelGGL((gla_kernel<T, DP, MODE, COLS>), dim3(units, a.H), dim3(threads), lds, s, a);
+  hipLaunchKernelGGL((gla_kernel<T, TO, DP, MODE, COLS>), dim3(units, a.H), dim3(threads), lds, s, a);
 }
 
 // A launch of MODE with ``cols`` columns of S a thread (1, 2 or 4; what DP allows is checked by the caller).
-template <typename T, int DP, int MODE>
+template <typename T, typename TO, int DP, int MODE>
 static void launch_gla_cols(const GlaArgs& a, int units, int cols, int threads, size_t lds, hipStream_t s) {
-  if constexpr (DP <= 16) { if (cols == 4) return launch_gla_mode<T, DP, MODE, 4>(a, units, threads, lds, s); }
-  if constexpr (DP <= 32) { if (cols == 2) return launch_gla_mode<T, DP, MODE, 2>(a, units, threads, lds, s); }
-  launch_gla_mode<T, DP, MODE, 1>(a, units, threads, lds, s);
+  if constexpr (DP <= 16) { if (cols == 4) return launch_gla_mode<T, TO, DP, MODE, 4>(a, units, threads, lds, s); }
+  if constexpr (DP <= 32) { if (cols == 2) return launch_gla_mode<T, TO, DP, MODE, 2>(a, units, threads, lds, s); }
+  launch_gla_mode<T, TO, DP, MODE, 1>(a, units, threads, lds, s);
 }
 
-template <typename T, int DP>
+template <typename T, typename TO, int DP>
 static int launch_gla(const GlaArgs& a, int R, int n_chunks, const int* req_chunk0, hipStream_t s) {
   // A thread holds 1, 2 or 4 columns of S as its registers allow (4 for runs of 16 channels, 2 for 32): what it reads of a
   // token's q, k and decays from LDS then serves several columns.  Two where possible (steps of single tokens, which are bound
@@ -241,21 +266,21 @@ static int launch_gla(const GlaArgs& a, int R, int n_chunks, const int* req_chun
               threads_for(cols_chunk), DP, GLA_MAX_THREADS(DP));
   const size_t lds = (size_t)STAGE * (4 * a.d + a.dv) * sizeof(float);
   if (n_chunks == 0) {
-    launch_gla_cols<T, DP, 0>(a, R, cols_walk, threads_for(cols_walk), lds, s);
+    launch_gla_cols<T, TO, DP, 0>(a, R, cols_walk, threads_for(cols_walk), lds, s);
     IFX_LAUNCH_CHECK();
   }
-  launch_gla_cols<T, DP, 1>(a, n_chunks, cols_chunk, threads_for(cols_chunk), lds, s);
+  launch_gla_cols<T, TO, DP, 1>(a, n_chunks, cols_chunk, threads_for(cols_chunk), lds, s);
   CombineArgs c{a.state, a.state_stride, a.state_offset, a.slots, req_chunk0, a.chunk_state, a.chunk_loga, a.H, a.d, a.dv, a.parts, DP};
   const size_t per = (size_t)a.H * a.dv * a.parts * DP;
   hipLaunchKernelGGL(gla_combine_kernel, dim3((unsigned)((per + 255) / 256), R), dim3(256), 0, s, c);
-  launch_gla_cols<T, DP, 2>(a, n_chunks, cols_chunk, threads_for(cols_chunk), lds, s);
+  launch_gla_cols<T, TO, DP, 2>(a, n_chunks, cols_chunk, threads_for(cols_chunk), lds, s);
   IFX_LAUNCH_CHECK();
 }
 
 // dp: channels a thread holds (16, 32, 64 or 128); parts: a power of two with parts * dp >= d; a head's columns, 1-4 a thread,
 // times parts must fit a workgroup.
-extern "C" int ifx_gla_scan(const void* rows, int dtype, int ld, int q_col, int k_col, int v_col, int g_col, const float* z,
-                            const float* z_bias, float inv_tau, float q_scale, float eps, const void* norm_w, int norm_dtype,
+extern "C" int ifx_gla_scan(const void* q, const void* k, const void* v, const void* g, int dtype, int out_dtype, int ld, const float* z,
+                            const float* z_bias, float inv_tau, float q_scale, float eps, const void* norm_w, int norm_dtype, const float* bonus,
                             float* state, long long state_stride, long long state_offset, const int* q_start, const int* q_len,
                             const int* slots, void* out, int T, int R, int H, int d, int dv, int dp, int parts,
                             int n_chunks, const int* chunk_req, const int* chunk_t0, const int* chunk_len,
@@ -267,15 +292,22 @@ extern "C" int ifx_gla_scan(const void* rows, int dtype, int ld, int q_col, int 
   IFX_REQUIRE(state_stride >= state_offset + (long long)H * dv * parts * dp, "gla_scan: a state row of %lld floats is too short", state_stride);
   IFX_REQUIRE(n_chunks == 0 || (chunk_req && chunk_t0 && chunk_len && req_chunk0 && chunk_state && chunk_loga), "gla_scan: chunks without their lists");
   IFX_REQUIRE((size_t)STAGE * (4 * d + dv) * sizeof(float) <= 64 * 1024, "gla_scan: d=%d, dv=%d need more LDS than a workgroup has", d, dv);
+  IFX_REQUIRE(!TIME_MIX || bonus, "time mixing needs the bonus per channel");
   if (T == 0 || R == 0) return 0;
-  GlaArgs a{rows, ld, q_col, k_col, v_col, g_col, z, z_bias, inv_tau, q_scale, eps, norm_w, norm_dtype, state,
+  GlaArgs a{q, k, v, g, ld, z, z_bias, inv_tau, q_scale, eps, norm_w, norm_dtype, bonus, state,
             (size_t)state_stride, (size_t)state_offset, q_start, q_len, slots, out, H, d, dv, parts,
             chunk_req, chunk_t0, chunk_len, chunk_state, chunk_loga};
   hipStream_t s = (hipStream_t)stream;
-#define GLA_CASE(TY, DPV) if (dp == DPV) return launch_gla<TY, DPV>(a, R, n_chunks, req_chunk0, s);
+#define GLA_CASE2(TY, TO, DPV) if (dp == DPV) return launch_gla<TY, TO, DPV>(a, R, n_chunks, req_chunk0, s);
+#define GLA_CASE(TY, DPV) GLA_CASE2(TY, TY, DPV)
+#if TIME_MIX
+  if (dtype == DT_F32 && out_dtype == DT_BF16) { GLA_CASE2(float, bf16_t, 16) GLA_CASE2(float, bf16_t, 32) GLA_CASE2(float, bf16_t, 64) GLA_CASE2(float, bf16_t, 128) }
+#endif
+  if (dtype != out_dtype) IFX_FAIL("gla_scan: rows of type %d with an output of type %d", dtype, out_dtype);
   if (dtype == DT_F32) { GLA_CASE(float, 16) GLA_CASE(float, 32) GLA_CASE(float, 64) GLA_CASE(float, 128) }
   else if (dtype == DT_BF16) { GLA_CASE(bf16_t, 16) GLA_CASE(bf16_t, 32) GLA_CASE(bf16_t, 64) GLA_CASE(bf16_t, 128) }
   else IFX_FAIL("gla_scan: unknown dtype %d", dtype);
 #undef GLA_CASE
+#undef GLA_CASE2
   IFX_FAIL("gla_scan: %d channels a thread (16, 32, 64 or 128)", dp);
 }

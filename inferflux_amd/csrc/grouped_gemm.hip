@@ -13,6 +13,8 @@
 //                      An expert from `n_real` upwards is an identity expert without weights: the first product leaves its
 //                      tiles alone and the second writes weight[item] * x[row] (`identity`, the rows as the first product
 //                      read them; N is then the rows' width).  The first product's activation is `act` of common.h.
+//                      With in_weights / weigh_input the weight is on the expert's input: the first product multiplies its sums
+//                      by it before the activation and the second leaves it out.
 //   ifx_headwise_grouped      out[t][h][:N] = W[h] x[t][h], tiles of TM rows of one head
 //
 // One kernel does all three products.  A workgroup of four waves takes TM = 64 or 128 items and TN = 128 weight rows;
@@ -97,6 +99,7 @@ struct GroupedArgs {
   int n_real;               // experts with weights; tiles of later ones are identity experts' (not MODE_HEADS)
   const bf16_t* identity;   // MODE_DOWN: [T][NW], what an identity expert hands back
   int act; float limit;     // MODE_GATE_UP: the activation
+  int weigh_input;          // the weight is on an expert's input: MODE_GATE_UP multiplies both sums by it, MODE_DOWN leaves it out
 };
 
 // MT: tiles of 32 items per wave (1: the workgroup takes 64 items, 2: 128)
@@ -202,6 +205,7 @@ __global__ __launch_bounds__(256) void grouped_kernel(GroupedArgs a) {
       // a tile of 32 weight rows is 16 of Wg and the same 16 of Wu: acc[i] (i < 8) is the gate of what acc[i + 8] is the up of
       const int ff = a.NW / 2;
       bf16_t* act = (bf16_t*)a.out + (size_t)m * ff;
+      const float wi = a.weigh_input ? a.weights[m] : 1.f;
 #pragma unroll
       for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
@@ -211,13 +215,13 @@ __global__ __launch_bounds__(256) void grouped_kernel(GroupedArgs a) {
           bf16x4 y;
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const float g = acc[mt][nt][4 * q + r], u = acc[mt][nt][8 + 4 * q + r];
+            const float g = wi * acc[mt][nt][4 * q + r], u = wi * acc[mt][nt][8 + 4 * q + r];
             y[r] = (__bf16)gated_act(g, u, a.act, a.limit);
           }
           *(bf16x4*)(act + f) = y;
         }
     } else {
-      const float wgt = MODE == MODE_DOWN ? a.weights[m] : 1.f;
+      const float wgt = MODE == MODE_DOWN && !a.weigh_input ? a.weights[m] : 1.f;
       float* of = MODE == MODE_DOWN ? (float*)a.out + ((size_t)(m % a.top) * a.T + m / a.top) * a.NW : nullptr;
       bf16_t* ob = MODE == MODE_HEADS ? (bf16_t*)a.out + ((size_t)m * a.n_groups + group) * a.out_head : nullptr;
       const bool whole4 = a.NW % 4 == 0 && (MODE == MODE_DOWN || a.out_head % 4 == 0);      // runs of four columns, stored at once
@@ -257,11 +261,11 @@ static int check_common(int K, int x_row, int x_group) {
 // act [n_items][ff] (bfloat16) from x [T][K] and the paired weights w [E][2 ff][K]; item i is row i / top.
 extern "C" int ifx_moe_gate_up_grouped(const void* x, const void* w, void* act, const int* sorted, const int* tile_expert,
                                        const int* tile_start, const int* tile_count, const int* n_tiles, int max_tiles, int tile_items,
-                                       int K, int ff, int top, int n_real, int act_kind, float limit, void* stream) {
+                                       int K, int ff, int top, int n_real, int act_kind, float limit, const float* in_weights, void* stream) {
   IFX_REQUIRE(check_common(K, K, 0) && ff > 0 && ff % 16 == 0 && top > 0, "moe_gate_up_grouped: K=%d must be a multiple of 8, ff=%d of 16", K, ff);
   if (max_tiles <= 0) return 0;
-  GroupedArgs a{(const bf16_t*)x, (const bf16_t*)w, act, sorted, tile_expert, tile_start, tile_count, n_tiles, nullptr,
-                K, 2 * ff, top, K, 0, 0, top, 0, 0, n_real, nullptr, act_kind, limit};
+  GroupedArgs a{(const bf16_t*)x, (const bf16_t*)w, act, sorted, tile_expert, tile_start, tile_count, n_tiles, in_weights,
+                K, 2 * ff, top, K, 0, 0, top, 0, 0, n_real, nullptr, act_kind, limit, in_weights ? 1 : 0};
   const dim3 grid(max_tiles, (2 * ff + TN - 1) / TN);
   if (tile_items == 128) hipLaunchKernelGGL((grouped_kernel<MODE_GATE_UP, 2>), grid, dim3(256), 0, (hipStream_t)stream, a);
   else if (tile_items == 64) hipLaunchKernelGGL((grouped_kernel<MODE_GATE_UP, 1>), grid, dim3(256), 0, (hipStream_t)stream, a);
@@ -273,11 +277,11 @@ extern "C" int ifx_moe_gate_up_grouped(const void* x, const void* w, void* act, 
 extern "C" int ifx_moe_down_grouped(const void* act, const void* w, float* parts, const float* weights, const int* sorted,
                                     const int* tile_expert, const int* tile_start, const int* tile_count, const int* n_tiles,
                                     int max_tiles, int tile_items, int T, int N, int ff, int top, int n_real, const void* identity,
-                                    void* stream) {
+                                    int weigh_input, void* stream) {
   IFX_REQUIRE(check_common(ff, ff, 0) && N > 0 && top > 0 && T >= 0, "moe_down_grouped: ff=%d must be a multiple of 8", ff);
   if (max_tiles <= 0 || T == 0) return 0;
   GroupedArgs a{(const bf16_t*)act, (const bf16_t*)w, parts, sorted, tile_expert, tile_start, tile_count, n_tiles, weights,
-                ff, N, 1, ff, 0, T, top, 0, 0, n_real, (const bf16_t*)identity, 0, 0.f};
+                ff, N, 1, ff, 0, T, top, 0, 0, n_real, (const bf16_t*)identity, 0, 0.f, weigh_input};
   const dim3 grid(max_tiles, (N + TN - 1) / TN);
   if (tile_items == 128) hipLaunchKernelGGL((grouped_kernel<MODE_DOWN, 2>), grid, dim3(256), 0, (hipStream_t)stream, a);
   else if (tile_items == 64) hipLaunchKernelGGL((grouped_kernel<MODE_DOWN, 1>), grid, dim3(256), 0, (hipStream_t)stream, a);
@@ -291,7 +295,7 @@ extern "C" int ifx_headwise_grouped(const void* x, const void* w, void* out, int
   IFX_REQUIRE(check_common(K, x_row, x_head) && N > 0 && H > 0 && out_head >= N, "headwise_grouped: K=%d, the rows of x (%d) and its heads (%d) must be multiples of 8", K, x_row, x_head);
   if (T <= 0) return 0;
   GroupedArgs a{(const bf16_t*)x, (const bf16_t*)w, out, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr,
-                K, N, 1, x_row, x_head, T, 1, out_head, H, H, nullptr, 0, 0.f};
+                K, N, 1, x_row, x_head, T, 1, out_head, H, H, nullptr, 0, 0.f, 0};
   if (T > 64) hipLaunchKernelGGL((grouped_kernel<MODE_HEADS, 2>), dim3(((T + 127) / 128) * H, (N + TN - 1) / TN), dim3(256), 0, (hipStream_t)stream, a);
   else hipLaunchKernelGGL((grouped_kernel<MODE_HEADS, 1>), dim3(((T + 63) / 64) * H, (N + TN - 1) / TN), dim3(256), 0, (hipStream_t)stream, a);
   IFX_LAUNCH_CHECK();

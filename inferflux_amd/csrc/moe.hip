@@ -8,6 +8,8 @@
 //                     s + choice_bias while the weights stay the scores s themselves.  Writes ids [T][top] (int32) and weights [T][top] (float), in
 //                     descending order of score, the lower index first among equals.
 //   ifx_moe_gate_up   a[t][j][:] = act(Wg[e] h_t, Wu[e] h_t) for e = ids[t][j]          (Wg, Wu [E][ff][K]; act: common.h)
+//                     With in_weights the activation reads in_weights[t][j] times both sums (the weight is on the expert's
+//                     input), and ifx_moe_down is told so (weigh_input: the experts' outputs are added as they are).
 //   ifx_moe_down      out[t][:] = sum_j weights[t][j] * Wd[e_j] a[t][j][:]              (Wd [E][N][ff])
 //                     An id from `n_real` upwards names an identity expert, which has no weights: its output is the
 //                     row h_t itself (ifx_moe_gate_up leaves such items alone, ifx_moe_down adds weights[t][j] * h_t).
@@ -199,7 +201,8 @@ template <typename T>
 __global__ __launch_bounds__(WAVE * WAVES) void moe_gate_up_kernel(const T* __restrict__ h, const T* __restrict__ wg,
                                                                    const T* __restrict__ wu, const int* __restrict__ ids,
                                                                    T* __restrict__ act, int K, int ff, int top, int paired,
-                                                                   int n_real, int act_kind, float limit) {
+                                                                   int n_real, int act_kind, float limit,
+                                                                   const float* __restrict__ in_weights) {
   const size_t item = blockIdx.x;                 // (row, choice)
   const size_t t = item / top;
   const int e = ids[item];
@@ -235,9 +238,10 @@ __global__ __launch_bounds__(WAVE * WAVES) void moe_gate_up_kernel(const T* __re
       sum[2 * r] = sg; sum[2 * r + 1] = su;
     }
   }
+  const float wi = in_weights ? in_weights[item] : 1.0f;      // a weight on the expert's input: on both sums, before the activation
 #pragma unroll
   for (int r = 0; r < ROWS_PER_WAVE; ++r) {
-    const float sg = wave_sum(sum[2 * r]), su = wave_sum(sum[2 * r + 1]);
+    const float sg = wi * wave_sum(sum[2 * r]), su = wi * wave_sum(sum[2 * r + 1]);
     if (lane == 0 && i0 + r < ff) act[item * ff + i0 + r] = from_f<T>(gated_act(sg, su, act_kind, limit));
   }
 }
@@ -246,7 +250,7 @@ template <typename T>
 __global__ __launch_bounds__(WAVE * WAVES) void moe_down_kernel(const T* __restrict__ act, const T* __restrict__ wd,
                                                                 const int* __restrict__ ids, const float* __restrict__ weights,
                                                                 T* __restrict__ out, int N, int ff, int top, int n_real,
-                                                                const T* __restrict__ h) {
+                                                                const T* __restrict__ h, int weigh_input) {
   const size_t t = blockIdx.x;
   const int wid = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int n0 = (blockIdx.y * WAVES + wid) * ROWS_PER_WAVE;
@@ -276,7 +280,7 @@ __global__ __launch_bounds__(WAVE * WAVES) void moe_down_kernel(const T* __restr
         sum[r] = s;
       }
     }
-    const float wj = weights[t * top + j];
+    const float wj = weigh_input ? 1.0f : weights[t * top + j];
 #pragma unroll
     for (int r = 0; r < ROWS_PER_WAVE; ++r) y[r] = fmaf(wj, wave_sum(sum[r]), y[r]);
   }
@@ -287,31 +291,31 @@ __global__ __launch_bounds__(WAVE * WAVES) void moe_down_kernel(const T* __restr
 }
 
 extern "C" int ifx_moe_gate_up(const void* h, const void* wg, const void* wu, const int* ids, void* act, int dtype, int T, int K,
-                               int ff, int top, int paired, int n_real, int act_kind, float limit, void* stream) {
+                               int ff, int top, int paired, int n_real, int act_kind, float limit, const float* in_weights, void* stream) {
   IFX_REQUIRE(T >= 0 && K > 0 && ff > 0 && top > 0, "moe_gate_up: bad sizes T=%d K=%d ff=%d top=%d", T, K, ff, top);
   IFX_REQUIRE(!paired || ff % 16 == 0, "moe_gate_up: paired weights need ff=%d to be a multiple of 16", ff);
   if (T == 0) return 0;
   const dim3 grid((unsigned)T * top, (ff + WAVES * ROWS_PER_WAVE - 1) / (WAVES * ROWS_PER_WAVE));
   hipStream_t s = (hipStream_t)stream;
   if (dtype == DT_F32)
-    hipLaunchKernelGGL(moe_gate_up_kernel<float>, grid, dim3(WAVE * WAVES), 0, s, (const float*)h, (const float*)wg, (const float*)wu, ids, (float*)act, K, ff, top, paired, n_real, act_kind, limit);
+    hipLaunchKernelGGL(moe_gate_up_kernel<float>, grid, dim3(WAVE * WAVES), 0, s, (const float*)h, (const float*)wg, (const float*)wu, ids, (float*)act, K, ff, top, paired, n_real, act_kind, limit, in_weights);
   else if (dtype == DT_BF16)
-    hipLaunchKernelGGL(moe_gate_up_kernel<bf16_t>, grid, dim3(WAVE * WAVES), 0, s, (const bf16_t*)h, (const bf16_t*)wg, (const bf16_t*)wu, ids, (bf16_t*)act, K, ff, top, paired, n_real, act_kind, limit);
+    hipLaunchKernelGGL(moe_gate_up_kernel<bf16_t>, grid, dim3(WAVE * WAVES), 0, s, (const bf16_t*)h, (const bf16_t*)wg, (const bf16_t*)wu, ids, (bf16_t*)act, K, ff, top, paired, n_real, act_kind, limit, in_weights);
   else IFX_FAIL("moe_gate_up: unknown dtype %d", dtype);
   IFX_LAUNCH_CHECK();
 }
 
 extern "C" int ifx_moe_down(const void* act, const void* wd, const int* ids, const float* weights, void* out, int dtype, int T,
-                            int N, int ff, int top, int n_real, const void* h, void* stream) {
+                            int N, int ff, int top, int n_real, const void* h, int weigh_input, void* stream) {
   IFX_REQUIRE(T >= 0 && N > 0 && ff > 0 && top > 0, "moe_down: bad sizes T=%d N=%d ff=%d top=%d", T, N, ff, top);
   IFX_REQUIRE(h != nullptr, "moe_down: the rows themselves are needed (identity experts read them)");
   if (T == 0) return 0;
   const dim3 grid(T, (N + WAVES * ROWS_PER_WAVE - 1) / (WAVES * ROWS_PER_WAVE));
   hipStream_t s = (hipStream_t)stream;
   if (dtype == DT_F32)
-    hipLaunchKernelGGL(moe_down_kernel<float>, grid, dim3(WAVE * WAVES), 0, s, (const float*)act, (const float*)wd, ids, weights, (float*)out, N, ff, top, n_real, (const float*)h);
+    hipLaunchKernelGGL(moe_down_kernel<float>, grid, dim3(WAVE * WAVES), 0, s, (const float*)act, (const float*)wd, ids, weights, (float*)out, N, ff, top, n_real, (const float*)h, weigh_input);
   else if (dtype == DT_BF16)
-    hipLaunchKernelGGL(moe_down_kernel<bf16_t>, grid, dim3(WAVE * WAVES), 0, s, (const bf16_t*)act, (const bf16_t*)wd, ids, weights, (bf16_t*)out, N, ff, top, n_real, (const bf16_t*)h);
+    hipLaunchKernelGGL(moe_down_kernel<bf16_t>, grid, dim3(WAVE * WAVES), 0, s, (const bf16_t*)act, (const bf16_t*)wd, ids, weights, (bf16_t*)out, N, ff, top, n_real, (const bf16_t*)h, weigh_input);
   else IFX_FAIL("moe_down: unknown dtype %d", dtype);
   IFX_LAUNCH_CHECK();
 }

@@ -75,6 +75,10 @@ class Model:
     def bind(self, tensors: Mapping[str, torch.Tensor], dtype: torch.dtype, device) -> "Model":
         for p in self.parts():
             p.load(tensors)
+        for j in self.injections[1:]:            # (the passes of a loop may read one matrix: one copy of it is enough)
+            share = getattr(j, "share_weights", None)
+            if share is not None and type(j) is type(self.injections[0]):
+                share(self.injections[0])
         self.dtype, self.device = dtype, torch.device(device)
         return self
 
@@ -122,7 +126,9 @@ class Model:
         for i, e in enumerate(schedule):
             block = self.blocks[e.layer]
             if e.before is not None:
-                self.injections[e.before].forward(residual, ctx, embedded)
+                if getattr(pending, "in_stream", False):
+                    pending = None
+                residual, pending = self.injections[e.before].apply(residual, pending, ctx, embedded)
             # a block that can hand on rows prepared for the next block's first norm is told that norm
             if i + 1 < len(schedule) and schedule[i + 1].before is not None:
                 following = None        # (the stream changes before that norm reads it)

@@ -43,6 +43,9 @@ TILE_QTS = (1, 2)
 DIRECT_TILE_HEAD_DIM = 128 if ARCH == "gfx950" else None
 
 
+TIME_MIX = (("TIME_MIX", 1),)           # the variant of gla.hip whose read-out comes before the write, with a bonus
+
+
 class KernelError(RuntimeError):
     pass
 
@@ -60,6 +63,10 @@ def module_variants() -> Iterable[Tuple[str, Variant]]:
     yield ("moe", ())
     yield ("ssm", ())
     yield ("gla", ())
+    yield ("gla", TIME_MIX)
+    yield ("time_mix", ())
+    yield ("matrix_memory", ())
+    yield ("deltas", ())
     yield ("delta", ())
     yield ("hyper", ())
     yield ("rowwise", ())
@@ -145,19 +152,19 @@ def embedding(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0) -> tor
 
 
 def embedding_scaled(ids: torch.Tensor, table: torch.Tensor, norm_weight: torch.Tensor, eps: float, scale: float = 1.0):
-    """``embedding`` (times ``scale``) for up to 16 tokens that also prepares the RMS norm (bfloat16 weight ``norm_weight`` [H]) which
+    """``embedding`` (times ``scale``) for up to 16 tokens that also prepares the RMS norm (weight ``norm_weight`` [H]) which
     reads the stream first: returns (the float32 stream [T, H], that norm's rows up to the factor per row)."""
     _check(ids, "ids", (None,), torch.int32)
     _check(table, "table", (None, None))
     T, H = ids.shape[0], table.shape[1]
-    _check(norm_weight, "norm_weight", (H,), torch.bfloat16)
+    _check(norm_weight, "norm_weight", (H,))
     if T > 16:
         raise KernelError(f"embedding_scaled: {T} rows (at most 16)")
     out = torch.empty((T, H), dtype=torch.float32, device=table.device)
     rows = torch.empty((T, H), dtype=torch.bfloat16, device=table.device)
     pieces = torch.empty((-(-H // 4096), 16), dtype=torch.float32, device=table.device)
-    _call(load_module("core"), "ifx_embedding_norm", (P, P, I, P, P, P, P, I, I, F, P),
-          ids.data_ptr(), table.data_ptr(), _dt(table), norm_weight.data_ptr(), out.data_ptr(), rows.data_ptr(),
+    _call(load_module("core"), "ifx_embedding_norm", (P, P, I, P, I, P, P, P, I, I, F, P),
+          ids.data_ptr(), table.data_ptr(), _dt(table), norm_weight.data_ptr(), _dt(norm_weight), out.data_ptr(), rows.data_ptr(),
           pieces.data_ptr(), T, H, float(scale), _stream())
     return out, ScaledRows(rows, pieces, H, eps, norm_weight)
 
@@ -167,12 +174,19 @@ def add_rmsnorm(residual: torch.Tensor, delta: Optional[torch.Tensor], weight: t
     """``residual`` [T, H] float32 (+= ``delta_scale`` * ``delta`` in place when given and no ``rows``), then RMSNorm.
 
     With ``rows`` (int32 [R]) only those rows are normalised, into [R, H], and the residual is
-    left untouched.
+    left untouched.  ``delta`` may also be ``SliceSums``, a ``ScaledDelta`` or a ``DeltaSum``.
     """
     _check(residual, "residual", (None, None), torch.float32)
     T, H = residual.shape
     _check(weight, "weight", (H,))
     n_slices = 1
+    if isinstance(delta, DeltaSum):
+        if delta_scale != 1.0:
+            delta = DeltaSum([(delta, delta_scale)])
+        if len(delta.terms) == 1 and not _is_vector(delta.terms[0][0]):
+            delta, delta_scale = delta.terms[0]
+        else:
+            return _add_terms_rmsnorm(residual, delta, weight, eps, out_dtype, rows)
     if isinstance(delta, ScaledDelta):             # a delta with its factor
         delta, delta_scale = delta.value, delta_scale * delta.scale
     if isinstance(delta, SliceSums):               # partial sums: the kernel adds them in slice order
@@ -189,6 +203,65 @@ def add_rmsnorm(residual: torch.Tensor, delta: Optional[torch.Tensor], weight: t
           residual.data_ptr(), _ptr(delta), _dt(delta) if delta is not None else 0, weight.data_ptr(),
           _dt(weight), out.data_ptr(), _DT[out_dtype], _ptr(rows), n, H, float(eps),
           1 if (delta is not None and rows is None) else 0, n_slices, T * H, float(delta_scale), _stream())
+    return out
+
+
+def _is_vector(t) -> bool:
+    return isinstance(t, torch.Tensor) and t.dim() == 1
+
+
+def _term_args(delta: "DeltaSum", T: int, H: int):
+    """(number of terms, pointers, dtypes, slices, slice strides, row strides, factors) as the kernels of deltas.hip take them."""
+    n = len(delta.terms)
+    if n > MAX_DELTA_TERMS:
+        raise KernelError(f"{n} additions at once (at most {MAX_DELTA_TERMS})")
+    rows = []
+    for v, scale in delta.terms:
+        if isinstance(v, SliceSums):
+            _check(v.parts, "delta", (None, T, H), torch.float32)
+            rows.append((v.parts.data_ptr(), DT_F32, v.parts.shape[0], T * H, H, scale))
+        else:
+            _check(v, "delta", (H,) if _is_vector(v) else (T, H))
+            rows.append((v.data_ptr(), _dt(v), 1, 0, 0 if _is_vector(v) else H, scale))
+    col = lambda c_type, i: (c_type * max(n, 1))(*[r[i] for r in rows])
+    return n, col(P, 0), col(I, 1), col(I, 2), col(LL, 3), col(I, 4), col(F, 5)
+
+
+MAX_DELTA_TERMS = 6
+_TERM_TYPES = (I, ctypes.POINTER(P), ctypes.POINTER(I), ctypes.POINTER(I), ctypes.POINTER(LL), ctypes.POINTER(I), ctypes.POINTER(F))
+
+
+def _add_terms_rmsnorm(residual, delta: "DeltaSum", weight, eps, out_dtype, rows):
+    T, H = residual.shape
+    n = T
+    if rows is not None:
+        _check(rows, "rows", (None,), torch.int32)
+        n = rows.shape[0]
+    out = torch.empty((n, H), dtype=out_dtype, device=residual.device)
+    _call(load_module("deltas"), "ifx_add_terms_rmsnorm", (P, *_TERM_TYPES, P, I, P, I, P, I, I, F, I, P),
+          residual.data_ptr(), *_term_args(delta, T, H), weight.data_ptr(), _dt(weight), out.data_ptr(), _DT[out_dtype], _ptr(rows), n, H,
+          float(eps), 0 if rows is not None else 1, _stream())
+    return out
+
+
+def join_stream(residual: torch.Tensor, delta, other: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+    """[T, 2 H] in ``dtype``: the stream ``residual`` [T, H] (float32) plus ``delta`` (anything ``add_rmsnorm`` takes, or None)
+    in the first H columns, ``other`` [T, H] (float32) in the rest.  The stream itself is left as it is."""
+    _check(residual, "residual", (None, None), torch.float32)
+    T, H = residual.shape
+    _check(other, "other", (T, H), torch.float32)
+    out = torch.empty((T, 2 * H), dtype=dtype, device=residual.device)
+    _call(load_module("deltas"), "ifx_join_stream", (P, *_TERM_TYPES, P, P, I, I, I, P),
+          residual.data_ptr(), *_term_args(DeltaSum.of(delta), T, H), other.data_ptr(), out.data_ptr(), _DT[dtype], T, H, _stream())
+    return out
+
+
+def query_temperature(positions: torch.Tensor, coef: float, every: int) -> torch.Tensor:
+    """float32 [T]: 1 + coef ln(floor((p + 1) / every) + 1) of int32 ``positions`` [T]."""
+    _check(positions, "positions", (None,), torch.int32)
+    out = torch.empty(positions.shape, dtype=torch.float32, device=positions.device)
+    _call(load_module("core"), "ifx_query_temperature", (P, P, I, F, I, P), positions.data_ptr(), out.data_ptr(), positions.shape[0],
+          float(coef), int(every), _stream())
     return out
 
 
@@ -210,12 +283,14 @@ def rope_append(qkv: torch.Tensor, bias: Optional[torch.Tensor], slots: Optional
                 k_cache: Optional[torch.Tensor], v_cache: Optional[torch.Tensor], page_size: int,
                 v_head_dim: Optional[int] = None, unit_norm_eps: Optional[float] = None, gate_out: Optional[torch.Tensor] = None,
                 v_first: Optional[torch.Tensor] = None, v_mix: float = 0.0, v_out: Optional[torch.Tensor] = None,
-                qk_norm: Optional[Tuple[torch.Tensor, torch.Tensor, float]] = None, extra_cols: int = 0) -> torch.Tensor:
+                qk_norm: Optional[Tuple[torch.Tensor, torch.Tensor, float]] = None, extra_cols: int = 0,
+                q_mult: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Bias, rotation and cache write of one step's projections; returns q [T, n_heads, head_dim].
 
     ``qk_norm`` (q weight [head_dim], k weight [head_dim], eps): before the rotation every q and k head becomes
     x / sqrt(mean(x^2) + eps) * weight.  ``extra_cols``: further columns at the end of every row of ``qkv`` that belong
-    to another kernel (a gate that is applied elsewhere).
+    to another kernel (a gate that is applied elsewhere).  ``q_mult`` float32 [T]: a factor on every query of a row, applied in
+    float before the rounding.
 
     Optionally: ``unit_norm_eps`` divides every q and k head by its root mean square (eps inside the root) after the
     rotation; ``gate_out`` (float32 [T, n_heads]) receives sigmoid(x + bias) of n_heads further columns behind q, k and v
@@ -259,15 +334,17 @@ def rope_append(qkv: torch.Tensor, bias: Optional[torch.Tensor], slots: Optional
         qn, kn, pre_eps = qk_norm
         _check(qn, "q norm weight", (head_dim,))
         _check(kn, "k norm weight", (head_dim,), qn.dtype)
+    if q_mult is not None:
+        _check(q_mult, "q_mult", (T,), torch.float32)
     q = torch.empty((T, n_heads, head_dim), dtype=dtype, device=qkv.device)
     _call(load_module("core"), "ifx_rope_append",
-          (P, I, P, I, P, P, P, I, I, I, I, I, I, I, P, P, P, I, LL, I, I, P, I, F, P, F, P, P, P, I, F, I, P),
+          (P, I, P, I, P, P, P, I, I, I, I, I, I, I, P, P, P, I, LL, I, I, P, I, F, P, F, P, P, P, I, F, I, P, P),
           qkv.data_ptr(), _DT[dtype], _ptr(bias), _dt(bias) if bias is not None else 0, _ptr(slots),
           _ptr(cos) if rope_style != ROPE_NONE else 0, _ptr(sin) if rope_style != ROPE_NONE else 0, rope_style,
           rotary_dim, T, n_heads, n_kv_heads, head_dim, page_size, q.data_ptr(), _ptr(k_cache), _ptr(v_cache),
           n_slices, T * width, dv, gate_cols, _ptr(gate_out), 1 if unit_norm_eps is not None else 0,
           float(unit_norm_eps or 0.0), _ptr(v_first), float(v_mix), _ptr(v_out), _ptr(qn), _ptr(kn),
-          _dt(qn) if qn is not None else 0, float(pre_eps) if qn is not None else 0.0, int(extra_cols), _stream())
+          _dt(qn) if qn is not None else 0, float(pre_eps) if qn is not None else 0.0, int(extra_cols), _ptr(q_mult), _stream())
     return q
 
 
@@ -289,6 +366,8 @@ def _delta_args(delta, shape, name):
     """(pointer, dtype code, slices, elements between slices) of a tensor or of a product left as ``SliceSums``."""
     if isinstance(delta, ScaledDelta):
         delta = delta.tensor()
+    if isinstance(delta, DeltaSum):
+        raise KernelError(f"{name}: several additions at once are the RMS norm's to add; form their sum first")
     if isinstance(delta, SliceSums):
         _check(delta.parts, name, (None, *shape), torch.float32)
         return delta.parts.data_ptr(), DT_F32, delta.parts.shape[0], delta.parts[0].numel()
@@ -304,6 +383,8 @@ def layernorm(x: torch.Tensor, delta, weight: torch.Tensor, eps: float, out_dtyp
     _check(x, "x", (None, None))
     T, H = x.shape
     _check(weight, "weight", (H,))
+    if isinstance(delta, DeltaSum):
+        delta = delta.tensor(x)
     dp, dd, n_slices, stride = (0, 0, 1, 0) if delta is None else _delta_args(delta, (T, H), "delta")
     n = T
     if rows is not None:
@@ -452,11 +533,13 @@ def pair_gate_up(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
 
 
 def moe_experts(h: torch.Tensor, gate: torch.Tensor, up: Optional[torch.Tensor], down: torch.Tensor, ids: torch.Tensor,
-                weights: torch.Tensor, act: int = ACT_SILU, limit: float = 0.0, n_identity: int = 0) -> torch.Tensor:
+                weights: torch.Tensor, act: int = ACT_SILU, limit: float = 0.0, n_identity: int = 0,
+                weigh_input: bool = False) -> torch.Tensor:
     """sum_j weights[t, j] * down[e] (act(gate[e] h_t, up[e] h_t)), e = ids[t, j], row by row: every (row, choice)
     streams its expert's weights (``gate`` / ``up`` [E, ff, K], or ``gate`` [E, 2 ff, K] from ``pair_gate_up`` and ``up``
     None; ``down`` [E, N, ff]; all in h's type).  With ``n_identity`` an id from E upwards names an identity expert, whose
-    output is the row itself (N = K then).  ``act``: ACT_SILU, ACT_GELU_TANH, or ACT_CLAMPED_SWISH with its ``limit``.  Returns [T, N]."""
+    output is the row itself (N = K then).  ``act``: ACT_SILU, ACT_GELU_TANH, or ACT_CLAMPED_SWISH with its ``limit``.  ``weigh_input``: the weights multiply the experts' inputs instead of their
+    outputs (in float, on the sums that the activation reads).  Returns [T, N]."""
     _check(h, "h", (None, None))
     T, K = h.shape
     paired = up is None
@@ -473,12 +556,12 @@ def moe_experts(h: torch.Tensor, gate: torch.Tensor, up: Optional[torch.Tensor],
         raise KernelError(f"moe_experts: identity experts hand back the row itself, so N={N} must equal K={K}")
     mod = load_module("moe")
     a = torch.empty((T, top, ff), dtype=h.dtype, device=h.device)
-    _call(mod, "ifx_moe_gate_up", (P, P, P, P, P, I, I, I, I, I, I, I, I, F, P),
+    _call(mod, "ifx_moe_gate_up", (P, P, P, P, P, I, I, I, I, I, I, I, I, F, P, P),
           h.data_ptr(), gate.data_ptr(), _ptr(up), ids.data_ptr(), a.data_ptr(), _dt(h), T, K, ff, top, 1 if paired else 0, E,
-          int(act), float(limit), _stream())
+          int(act), float(limit), weights.data_ptr() if weigh_input else 0, _stream())
     out = torch.empty((T, N), dtype=h.dtype, device=h.device)
-    _call(mod, "ifx_moe_down", (P, P, P, P, P, I, I, I, I, I, I, P, P),
-          a.data_ptr(), down.data_ptr(), ids.data_ptr(), weights.data_ptr(), out.data_ptr(), _dt(h), T, N, ff, top, E, h.data_ptr(), _stream())
+    _call(mod, "ifx_moe_down", (P, P, P, P, P, I, I, I, I, I, I, P, I, P),
+          a.data_ptr(), down.data_ptr(), ids.data_ptr(), weights.data_ptr(), out.data_ptr(), _dt(h), T, N, ff, top, E, h.data_ptr(), 1 if weigh_input else 0, _stream())
     return out
 
 
@@ -494,12 +577,13 @@ def grouped_takes(dtype: torch.dtype, K: int, ff: int) -> bool:
 
 
 def moe_experts_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, ids: torch.Tensor,
-                        weights: torch.Tensor, act: int = ACT_SILU, limit: float = 0.0, n_identity: int = 0) -> "SliceSums":
+                        weights: torch.Tensor, act: int = ACT_SILU, limit: float = 0.0, n_identity: int = 0,
+                        weigh_input: bool = False) -> "SliceSums":
     """The same sum for steps of many rows, on the matrix cores: the (row, choice) items are ordered by expert on the
     device and every expert's weights meet tiles of its items (bfloat16; ``gate_up`` from ``pair_gate_up``).  Returns the
     choices' weighted outputs as ``SliceSums`` [top, T, N] (float32), which the kernel that adds them to the stream sums
     in the order of the choices.  ``n_identity``: ids from E up to E + n_identity name identity experts, whose output is
-    the row itself (N = K then); ``act`` and ``limit`` as for ``moe_experts``."""
+    the row itself (N = K then); ``act``, ``limit`` and ``weigh_input`` as for ``moe_experts``."""
     _check(h, "h", (None, None), torch.bfloat16)
     T, K = h.shape
     _check(gate_up, "gate_up", (None, None, K), torch.bfloat16)
@@ -523,13 +607,15 @@ def moe_experts_grouped(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tens
     _call(mod, "ifx_moe_sort", (P, I, I, I, P, P, P, P, P, P), ids.data_ptr(), n_items, E, tile_items, sorted_.data_ptr(), te.data_ptr(),
           ts.data_ptr(), tc.data_ptr(), nt.data_ptr(), _stream())
     a = torch.empty((n_items, ff), dtype=torch.bfloat16, device=h.device)
-    _call(mod, "ifx_moe_gate_up_grouped", (P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P),
+    _call(mod, "ifx_moe_gate_up_grouped", (P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, F, P, P),
           h.data_ptr(), gate_up.data_ptr(), a.data_ptr(), sorted_.data_ptr(), te.data_ptr(), ts.data_ptr(), tc.data_ptr(),
-          nt.data_ptr(), max_tiles, tile_items, K, ff, top, n_real, int(act), float(limit), _stream())
+          nt.data_ptr(), max_tiles, tile_items, K, ff, top, n_real, int(act), float(limit),
+          weights.data_ptr() if weigh_input else 0, _stream())
     parts = torch.empty((top, T, N), dtype=torch.float32, device=h.device)
-    _call(mod, "ifx_moe_down_grouped", (P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, P),
+    _call(mod, "ifx_moe_down_grouped", (P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P, I, P),
           a.data_ptr(), down.data_ptr(), parts.data_ptr(), weights.data_ptr(), sorted_.data_ptr(), te.data_ptr(), ts.data_ptr(),
-          tc.data_ptr(), nt.data_ptr(), max_tiles, tile_items, T, N, ff, top, n_real, h.data_ptr(), _stream())
+          tc.data_ptr(), nt.data_ptr(), max_tiles, tile_items, T, N, ff, top, n_real, h.data_ptr(), 1 if weigh_input else 0,
+          _stream())
     return SliceSums(parts, torch.bfloat16)
 
 
@@ -642,6 +728,16 @@ class LinearWeight:
     def dtype(self):
         return self.rows.dtype
 
+    def part(self, start: int, stop: int) -> "LinearWeight":
+        """Rows ``start`` .. ``stop`` - 1 as a weight of their own, sharing this one's memory (the copy too, where whole
+        tiles of it hold just these rows)."""
+        N, K = self.rows.shape
+        tiled, tr = None, self.tile_rows
+        if self.tiled is not None and self.order is None and start % tr == 0 and (stop % tr == 0 or stop == N):
+            per_tile = tr * (-(-K // 64) * 64)
+            tiled = self.tiled[start // tr * per_tile:-(-stop // tr) * per_tile]
+        return LinearWeight(self.rows[start:stop], tiled, None, tr if tiled is not None else 16)
+
 
 # Whether prepare_linear makes tiled copies, and how much memory it leaves free when it does.
 decode_weight_copy = True
@@ -709,6 +805,37 @@ class ScaledDelta:
         return v * self.scale
 
 
+class DeltaSum:
+    """Several things to be added to the stream, each times a factor: ``terms`` is a list of (value, factor), a value being a
+    tensor [T, H], ``SliceSums`` or one vector [H] for all rows.  ``add_rmsnorm`` takes it as its delta and ``join_stream``
+    as what is pending; nested sums and ``ScaledDelta`` are taken apart."""
+
+    __slots__ = ("terms",)
+
+    def __init__(self, terms):
+        flat = []
+        for v, s in terms:
+            if isinstance(v, DeltaSum):
+                flat += [(w, s * t) for w, t in v.terms]
+            elif isinstance(v, ScaledDelta):
+                flat.append((v.value, s * v.scale))
+            else:
+                flat.append((v, float(s)))
+        self.terms = flat
+
+    @classmethod
+    def of(cls, *values) -> "DeltaSum":
+        """The sum of ``values`` (None: nothing), each with factor 1."""
+        return cls([(v, 1.0) for v in values if v is not None])
+
+    def tensor(self, like: torch.Tensor) -> torch.Tensor:
+        """The sum as a float32 tensor of ``like``'s shape (for readers that add one tensor)."""
+        out = torch.zeros_like(like, dtype=torch.float32)
+        for v, s in self.terms:
+            out += (v.sum(torch.float32) if isinstance(v, SliceSums) else v.float()) * s
+        return out
+
+
 class SliceSums:
     """A product left as partial sums over slices of K: it stands for ``parts.sum(0)`` (float32 [S, M, N], added in
     slice order).  ``add_rmsnorm`` takes it as its delta and ``rope_append`` as its q/k/v, which saves the kernel
@@ -760,32 +887,33 @@ def adds_into_stream(n_rows: int, weight, norm_weight: torch.Tensor) -> bool:
     N, K = weight.rows.shape
     if norm_weight is None:           # (a reader that takes partial sums but keeps the addition to itself)
         return False
-    return (weight.rows.dtype == torch.bfloat16 and norm_weight.dtype == torch.bfloat16 and n_rows <= 16 and N % 4 == 0
+    return (weight.rows.dtype == torch.bfloat16 and n_rows <= 16 and N % 4 == 0
             and _small_m_kernel(n_rows, N, K, weight.tiled is not None) == "skinny")
 
 
 def linear_into_stream(x: torch.Tensor, weight: LinearWeight, stream: torch.Tensor, norm_weight: torch.Tensor,
                        eps: float, mult: float = 1.0) -> ScaledRows:
     """``stream`` [M <= 16, N] (float32) += ``mult`` * x [M, K] W^T in place, as the product's epilogue, which also prepares
-    the RMS norm that follows (weight ``norm_weight`` [N] bfloat16): returns its rows up to the factor per row."""
+    the RMS norm that follows (weight ``norm_weight`` [N]): returns its rows up to the factor per row."""
     _check(x, "x", (None, None), torch.bfloat16)
     M, K = x.shape
     N = weight.rows.shape[0]
     if not adds_into_stream(M, weight, norm_weight) or weight.rows.shape[1] != K:
         raise KernelError(f"linear_into_stream: not for {M} rows times a {tuple(weight.rows.shape)} weight")
     _check(stream, "stream", (M, N), torch.float32)
-    _check(norm_weight, "norm_weight", (N,), torch.bfloat16)
+    _check(norm_weight, "norm_weight", (N,))
     rows = torch.empty((M, N), dtype=torch.bfloat16, device=x.device)
     tile_rows = 16 if weight.tiled is None else weight.tile_rows
     pieces = torch.empty((-(-N // tile_rows), 16), dtype=torch.float32, device=x.device)    # one piece per row tile
     w = weight.rows if weight.tiled is None else weight.tiled
     _call(load_module("gemm_bf16"), "ifx_skinny_gemm", _SKINNY_ARGS,
           x.data_ptr(), w.data_ptr(), 0, DT_F32, M, N, K, 0, 0, 0, 2, 0 if weight.tiled is None else tile_rows, 0,
-          0, 0, 0.0, 0.0, stream.data_ptr(), norm_weight.data_ptr(), rows.data_ptr(), pieces.data_ptr(), float(mult), _stream())
+          0, 0, 0.0, 0.0, stream.data_ptr(), norm_weight.data_ptr(), 1 if norm_weight.dtype == torch.float32 else 0, rows.data_ptr(),
+          pieces.data_ptr(), float(mult), 0, 0, _stream())
     return ScaledRows(rows, pieces, N, eps, norm_weight)
 
 
-_SKINNY_ARGS = (P, P, P, I, I, I, I, I, I, I, I, I, P, P, I, F, F, P, P, P, P, F, P)
+_SKINNY_ARGS = (P, P, P, I, I, I, I, I, I, I, I, I, P, P, I, F, F, P, P, I, P, P, F, I, I, P)
 
 
 def pair_tile_order(n_heads: int, head_dim: int) -> list:
@@ -856,8 +984,8 @@ def skinny_gemm(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = 
         raise KernelError("skinny_gemm: a tile order goes with a tiled copy and a plain product")
     _call(load_module("gemm_bf16"), "ifx_skinny_gemm", _SKINNY_ARGS,
           x.data_ptr(), (weight if tiled is None else tiled).data_ptr(), out.data_ptr(), _DT[out_dtype], M, N, K, nt, waves,
-          unroll, _GATED_EPILOGUE[act] if swiglu_pairs else 0, 0 if tiled is None else tile_rows, _ptr(order), *scale, 0, 0, 0, 0,
-          1.0, _stream())
+          unroll, _GATED_EPILOGUE[act] if swiglu_pairs else 0, 0 if tiled is None else tile_rows, _ptr(order), *scale, 0, 0, 0, 0, 0,
+          1.0, 0, 0, _stream())
     return out
 
 
@@ -886,10 +1014,61 @@ def wide_gemm(x, weight: LinearWeight, out_dtype: torch.dtype = torch.bfloat16, 
     part = torch.empty((n_slices, M, N), dtype=torch.float32, device=x.device) if n_slices > 1 else None
     keep = keep_slices and n_slices > 1
     out = None if keep else torch.empty((M, N // 2 if swiglu_pairs else N), dtype=out_dtype, device=x.device)
-    _call(mod, "ifx_wide_gemm", (P, P, P, I, P, I, I, I, I, I, I, P, I, P, I, F, F, P),
+    _call(mod, "ifx_wide_gemm", (P, P, P, I, P, I, I, I, I, I, I, P, I, P, I, F, F, I, I, P),
           x.data_ptr(), weight.tiled.data_ptr(), _ptr(out), _DT[out_dtype], _ptr(part), M, N, K, n_waves, n_slices,
-          _GATED_EPILOGUE[act] if swiglu_pairs else 0, _ptr(weight.order), weight.tile_rows, *scale, _stream())
+          _GATED_EPILOGUE[act] if swiglu_pairs else 0, _ptr(weight.order), weight.tile_rows, *scale, 0, 0, _stream())
     return SliceSums(part, out_dtype) if keep else out
+
+
+def streams_weight(n_rows: int, weight) -> bool:
+    """Whether ``linear`` of ``n_rows`` rows with this weight goes to the kernels that stream a weight for few rows (whose
+    float sums cost nothing more than rounded ones) or, in 32-bit, to the 32-bit kernel, and not to the library."""
+    rows = weight.rows if isinstance(weight, LinearWeight) else weight
+    if rows.dtype == torch.float32:
+        return True
+    has_tiled = isinstance(weight, LinearWeight) and weight.tiled is not None
+    return _small_m_kernel(n_rows, rows.shape[0], rows.shape[1], has_tiled) is not None
+
+
+def _blocks_kernel(n_rows: int, weight, block_rows: int) -> Optional[str]:
+    if not (isinstance(weight, LinearWeight) and weight.dtype == torch.bfloat16 and weight.tiled is not None and weight.order is None
+            and weight.tile_rows == 16 and block_rows % 16 == 0 and weight.rows.shape[1] % 8 == 0):
+        return None
+    if n_rows <= 16:
+        return "skinny"
+    return "wide" if n_rows <= SKINNY_MAX_M and block_rows % 128 == 0 else None
+
+
+def takes_blocks(n_rows: int, weight, block_rows: int) -> bool:
+    """Whether ``linear_blocks`` takes this shape."""
+    return _blocks_kernel(n_rows, weight, block_rows) is not None
+
+
+def linear_blocks(x: torch.Tensor, weight: "LinearWeight", block_rows: int, out_dtype: torch.dtype = torch.bfloat16) -> torch.Tensor:
+    """Several products of few rows in one launch: ``x`` [n, M, K] holds n inputs, ``weight`` [N, K] (with its copy in tiles of
+    16 rows) n blocks of rows, all of ``block_rows`` except the last, which is what remains; block b's columns of the result
+    [M, N] are x[b] times block b transposed."""
+    _check(x, "x", (None, None, None), torch.bfloat16)
+    n, M, K = x.shape
+    kind = _blocks_kernel(M, weight, block_rows)
+    N = weight.rows.shape[0]
+    if kind is None or weight.rows.shape[1] != K or not (n - 1) * block_rows < N:
+        raise KernelError(f"linear_blocks: not for {n} inputs of {M} rows times a {tuple(weight.rows.shape)} weight in blocks of {block_rows}")
+    tiles = block_rows // 16
+    if kind == "skinny":
+        out = torch.empty((M, N), dtype=out_dtype, device=x.device)
+        _call(load_module("gemm_bf16"), "ifx_skinny_gemm", _SKINNY_ARGS, x.data_ptr(), weight.tiled.data_ptr(), out.data_ptr(), _DT[out_dtype],
+              M, N, K, 0 if tiles % 2 == 0 else 1, 0, 0, 0, 16, 0, 0, 0, 0.0, 0.0, 0, 0, 0, 0, 0, 1.0, tiles, n, _stream())
+        return out
+    mod = load_module("gemm_wide")
+    plan = mod.fn("ifx_wide_gemm_plan", (I, I, I, I, I, I, I))(M, N, K, 8, 0, 0, 16)
+    n_slices = plan % 256
+    part = torch.empty((n_slices, M, N), dtype=torch.float32, device=x.device) if n_slices > 1 else None
+    out = torch.empty((M, N), dtype=out_dtype, device=x.device)
+    _call(mod, "ifx_wide_gemm", (P, P, P, I, P, I, I, I, I, I, I, P, I, P, I, F, F, I, I, P),
+          x.data_ptr(), weight.tiled.data_ptr(), out.data_ptr(), _DT[out_dtype], _ptr(part), M, N, K, 8, n_slices, 0, 0, 16, 0, 0, 0.0, 0.0,
+          tiles, n, _stream())
+    return out
 
 
 def staged_gemm(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = torch.bfloat16,
@@ -1382,23 +1561,183 @@ def gla_scan(rows: torch.Tensor, cols: Tuple[int, int, int, int], z: torch.Tenso
     for t, nm in ((q_start, "q_start"), (q_len, "q_len"), (slots, "slots")):
         _check(t, nm, (R,), torch.int32)
     dp, parts = gla_layout(d, dv)
+    if state_offset + n_heads * dv * parts * dp > state.shape[1]:
+        raise KernelError("gla_scan: the state rows are too short")
     out = torch.empty((T, HV), dtype=rows.dtype, device=rows.device)
-    n_chunks, lists = 0, (0, 0, 0, 0, 0, 0)
-    if chunks is not None:
-        n_chunks = chunks["req"].shape[0]
-        for nm in ("req", "t0", "len"):
-            _check(chunks[nm], f"chunks.{nm}", (n_chunks,), torch.int32)
-        _check(chunks["req_chunk0"], "chunks.req_chunk0", (R + 1,), torch.int32)
-        chunk_state = torch.empty((n_chunks, HV * parts * dp), dtype=torch.float32, device=rows.device)
-        chunk_loga = torch.empty((n_chunks, HD), dtype=torch.float32, device=rows.device)
-        lists = (chunks["req"].data_ptr(), chunks["t0"].data_ptr(), chunks["len"].data_ptr(), chunks["req_chunk0"].data_ptr(),
-                 chunk_state.data_ptr(), chunk_loga.data_ptr())
-    _call(load_module("gla"), "ifx_gla_scan",
-          (P, I, I, I, I, I, I, P, P, F, F, F, P, I, P, LL, LL, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P, P, P, P, P),
-          rows.data_ptr(), _dt(rows), ld, q_col, k_col, v_col, g_col, z.data_ptr(), _ptr(z_bias), 1.0 / float(tau), float(q_scale),
-          float(eps), norm_weight.data_ptr(), _dt(norm_weight), state.data_ptr(), state.shape[1], int(state_offset),
-          q_start.data_ptr(), q_len.data_ptr(), slots.data_ptr(), out.data_ptr(), T, R, n_heads, d, dv, dp, parts, n_chunks,
-          *lists, _stream())
+    base, size = rows.data_ptr(), rows.element_size()
+    n_chunks, lists, _keep = _chunk_lists(chunks, R, HV * parts * dp, HD, rows.device)
+    _call(load_module("gla"), "ifx_gla_scan", _GLA_ARGS,
+          base + q_col * size, base + k_col * size, base + v_col * size, base + g_col * size, _dt(rows), _dt(out), ld, z.data_ptr(),
+          _ptr(z_bias), 1.0 / float(tau), float(q_scale), float(eps), norm_weight.data_ptr(), _dt(norm_weight), 0, state.data_ptr(),
+          state.shape[1], int(state_offset), q_start.data_ptr(), q_len.data_ptr(), slots.data_ptr(), out.data_ptr(), T, R, n_heads, d, dv,
+          dp, parts, n_chunks, *lists, _stream())
+    return out
+
+
+_GLA_ARGS = (P, P, P, P, I, I, I, P, P, F, F, F, P, I, P, P, LL, LL, P, P, P, P, I, I, I, I, I, I, I, I, P, P, P, P, P, P, P)
+
+
+def _chunk_lists(chunks: Optional[Dict[str, object]], R: int, state_floats: int, log_floats: int, device):
+    """(number of chunks, the kernel's list arguments, what they point into) of ``gla_scan`` and ``time_mix_scan``."""
+    if chunks is None:
+        return 0, (0, 0, 0, 0, 0, 0), None
+    n_chunks = chunks["req"].shape[0]
+    for nm in ("req", "t0", "len"):
+        _check(chunks[nm], f"chunks.{nm}", (n_chunks,), torch.int32)
+    _check(chunks["req_chunk0"], "chunks.req_chunk0", (R + 1,), torch.int32)
+    chunk_state = torch.empty((n_chunks, state_floats), dtype=torch.float32, device=device)
+    chunk_loga = torch.empty((n_chunks, log_floats), dtype=torch.float32, device=device)
+    return n_chunks, (chunks["req"].data_ptr(), chunks["t0"].data_ptr(), chunks["len"].data_ptr(), chunks["req_chunk0"].data_ptr(),
+                      chunk_state.data_ptr(), chunk_loga.data_ptr()), (chunk_state, chunk_loga)
+
+
+def _check_rows(t: torch.Tensor, name: str, T: int, width: int, dtype: Optional[torch.dtype] = None) -> int:
+    """``t`` [T, width] on the GPU with contiguous rows that may lie further apart; returns their distance."""
+    if not (isinstance(t, torch.Tensor) and t.is_cuda and tuple(t.shape) == (T, width) and (dtype is None or t.dtype == dtype)
+            and (width == 1 or t.stride(1) == 1) and (T <= 1 or t.stride(0) >= width)):
+        raise KernelError(f"{name}: needs [{T}, {width}] rows on the GPU" + (f" of {dtype}" if dtype is not None else ""))
+    return t.stride(0) if T > 1 else max(t.stride(0), width)
+
+
+def shifted_mixes(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, state_offset: int, row_req: torch.Tensor, q_start: torch.Tensor,
+                  q_len: torch.Tensor, slots: torch.Tensor) -> torch.Tensor:
+    """[S, T, H] in h's type: h + (h' - h) mu[s] with h' the request's row before, ``mu`` float32 [S, H].  A request's last row lives
+    in the H floats from ``state_offset`` of its row of ``state`` [slots, n] (float32, zero for a request that starts): it is
+    read as the row before this step's first and replaced by this step's last."""
+    _check(h, "h", (None, None))
+    T, H = h.shape
+    _check(mu, "mu", (None, H), torch.float32)
+    _check(state, "state", (None, None), torch.float32)
+    _check(row_req, "row_req", (T,), torch.int32)
+    R = q_start.shape[0]
+    for t, nm in ((q_start, "q_start"), (q_len, "q_len"), (slots, "slots")):
+        _check(t, nm, (R,), torch.int32)
+    out = torch.empty((mu.shape[0], T, H), dtype=h.dtype, device=h.device)
+    _call(load_module("time_mix"), "ifx_shifted_mixes", (P, I, P, P, LL, LL, P, P, P, P, P, I, I, I, P),
+          h.data_ptr(), _dt(h), mu.data_ptr(), state.data_ptr(), state.shape[1], int(state_offset), row_req.data_ptr(), q_start.data_ptr(),
+          q_len.data_ptr(), slots.data_ptr(), out.data_ptr(), T, H, mu.shape[0], _stream())
+    return out
+
+
+def lowrank_tanh(a: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """tanh(a) W^T in float: ``a`` float32 [T, r] (rows may lie further apart), ``w`` [C, r]; float32 [T, C]."""
+    _check(w, "w", (None, None))
+    C, r = w.shape
+    T = a.shape[0]
+    lda = _check_rows(a, "a", T, r, torch.float32)
+    z = torch.empty((T, C), dtype=torch.float32, device=w.device)
+    _call(load_module("time_mix"), "ifx_lowrank_tanh", (P, I, P, I, P, I, I, I, P), a.data_ptr(), lda, w.data_ptr(), _dt(w), z.data_ptr(), T, r, C,
+          _stream())
+    return z
+
+
+def time_mix_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, g: torch.Tensor, z: torch.Tensor, w0: torch.Tensor, u: torch.Tensor,
+                  norm_weight: torch.Tensor, eps: float, n_heads: int, d: int, state: torch.Tensor, state_offset: int, q_start: torch.Tensor,
+                  q_len: torch.Tensor, slots: torch.Tensor, out_dtype: torch.dtype, chunks: Optional[Dict[str, object]] = None) -> torch.Tensor:
+    """Time mixing's recurrence over each request's rows, with the output's norm and gate: w = exp(-exp(z + w0)) per key channel;
+    o = (S + diag(u) k v^T)^T r; S <- diag(w) S + k v^T; y = o / sqrt(mean(o^2) + eps) * norm_weight * silu(g).  ``r``, ``k``,
+    ``v``, ``g`` [T, n_heads * d] (one element type; rows equally far apart), ``z`` float32 [T, n_heads * d], ``w0`` float32
+    [n_heads * d], ``u`` float32 [n_heads, d], ``norm_weight`` float32 [n_heads * d]; ``state`` as for ``gla_scan`` (values as
+    wide as keys), and ``chunks`` too.  Everything between is float.  Returns y [T, n_heads * d] in ``out_dtype``."""
+    T, HD = r.shape[0], n_heads * d
+    lds = [_check_rows(t, nm, T, HD, r.dtype) for t, nm in ((r, "r"), (k, "k"), (v, "v"), (g, "g"))]
+    if len(set(lds)) != 1:
+        raise KernelError(f"time_mix_scan: rows {lds} elements apart (they must agree)")
+    _check(z, "z", (T, HD), torch.float32)
+    for t, nm, shape in ((w0, "w0", (HD,)), (u, "u", (n_heads, d)), (norm_weight, "norm_weight", (HD,))):
+        _check(t, nm, shape, torch.float32)
+    _check(state, "state", (None, None), torch.float32)
+    R = q_start.shape[0]
+    for t, nm in ((q_start, "q_start"), (q_len, "q_len"), (slots, "slots")):
+        _check(t, nm, (R,), torch.int32)
+    dp, parts = gla_layout(d, d)
+    if state_offset + HD * parts * dp > state.shape[1]:
+        raise KernelError("time_mix_scan: the state rows are too short")
+    out = torch.empty((T, HD), dtype=out_dtype, device=r.device)
+    n_chunks, lists, _keep = _chunk_lists(chunks, R, HD * parts * dp, HD, r.device)
+    _call(load_module("gla", TIME_MIX), "ifx_gla_scan", _GLA_ARGS,
+          r.data_ptr(), k.data_ptr(), v.data_ptr(), g.data_ptr(), _dt(r), _DT[out_dtype], lds[0], z.data_ptr(), w0.data_ptr(), 1.0, 1.0,
+          float(eps), norm_weight.data_ptr(), _dt(norm_weight), u.data_ptr(), state.data_ptr(), state.shape[1], int(state_offset),
+          q_start.data_ptr(), q_len.data_ptr(), slots.data_ptr(), out.data_ptr(), T, R, n_heads, d, d, dp, parts, n_chunks, *lists, _stream())
+    return out
+
+
+# ----------------------------------------------------------------------------------------
+MEMORY_THREAD_CHANNELS = (4, 8, 16, 32)     # key channels of a column of S a thread may hold
+MEMORY_MAX_PADDED_DIM, MEMORY_THREADS = 512, 256
+
+
+def matrix_memory_layout(d: int, dv: int, single_tokens: bool = False) -> Tuple[int, int, int]:
+    """(channels a thread, threads a column, columns a workgroup) of the matrix memory's walk for heads of ``d`` key channels
+    and ``dv`` values (dv + 1 columns: the last is the normaliser's), the columns dealt evenly to as many workgroups as it takes.
+    The state's layout (columns of d padded to a power of two) does not depend on the choice: a walk over many tokens is
+    shortest with few channels a thread, steps of single tokens want few workgroups (``single_tokens``)."""
+    dpad = 4
+    while dpad < d:
+        dpad *= 2
+    if dpad > MEMORY_MAX_PADDED_DIM:
+        raise KernelError(f"matrix memory: heads of {d} key channels (at most {MEMORY_MAX_PADDED_DIM})")
+    found = [(ch, dpad // ch) for ch in MEMORY_THREAD_CHANNELS if ch <= dpad and dpad // ch <= 64]
+    ch, ks = found[0]
+    if single_tokens:
+        ch, ks = next((f for f in reversed(found) if f[0] <= 16), found[0])
+    most = max(1, MEMORY_THREADS // ks)
+    groups = -(-(dv + 1) // most)
+    return ch, ks, -(-(dv + 1) // groups)
+
+
+def _memory_max_floats(n_heads: int) -> int:
+    return -(-n_heads // 4) * 4         # the running maxima come first in a state row
+
+
+def matrix_memory_state_floats(n_heads: int, d: int, dv: int) -> int:
+    ch, ks, _ = matrix_memory_layout(d, dv)
+    return _memory_max_floats(n_heads) + n_heads * (dv + 1) * ch * ks
+
+
+def matrix_memory(rows: torch.Tensor, cols: Tuple[int, int, int, int], gates: torch.Tensor, gate_cols: Tuple[int, int], i_bias: torch.Tensor,
+                  f_bias: torch.Tensor, cap: float, norm_weight: torch.Tensor, eps: float, n_heads: int, d: int, dv: int, state: torch.Tensor,
+                  q_start: torch.Tensor, q_len: torch.Tensor, slots: torch.Tensor, row_req: torch.Tensor, out_dtype: torch.dtype,
+                  single_tokens: bool = False) -> torch.Tensor:
+    """Matrix memory with exponential gates over each request's rows, with the output's norm and gate (see
+    csrc/matrix_memory.hip).  ``rows`` [T, ld] holds q, k (n_heads * d each), v and the output gate (n_heads * dv each) at the
+    columns ``cols``; ``gates`` float32 [T, ldg] the input and forget gates' numbers (n_heads each) at ``gate_cols``; biases
+    float32 [n_heads], ``norm_weight`` float32 [n_heads * dv].  ``state`` float32 [slots, ``matrix_memory_state_floats``], zero
+    for a request that starts.  ``single_tokens``: every request brings one row.  Returns [T, n_heads * dv] in ``out_dtype``."""
+    _check(rows, "rows", (None, None))
+    T, ld = rows.shape
+    _check(gates, "gates", (T, None), torch.float32)
+    ldg = gates.shape[1]
+    HD, HV = n_heads * d, n_heads * dv
+    q_col, k_col, v_col, g_col = (int(c) for c in cols)
+    for c, w, nm in ((q_col, HD, "q"), (k_col, HD, "k"), (v_col, HV, "v"), (g_col, HV, "gate")):
+        if c < 0 or c + w > ld:
+            raise KernelError(f"matrix_memory: the {nm} columns {c}..{c + w} lie outside rows of {ld}")
+    i_col, f_col = (int(c) for c in gate_cols)
+    if min(i_col, f_col) < 0 or max(i_col, f_col) + n_heads > ldg:
+        raise KernelError(f"matrix_memory: the gates' columns {i_col}, {f_col} lie outside rows of {ldg}")
+    for t, nm, shape in ((i_bias, "i_bias", (n_heads,)), (f_bias, "f_bias", (n_heads,)), (norm_weight, "norm_weight", (HV,))):
+        _check(t, nm, shape, torch.float32)
+    _check(state, "state", (None, None), torch.float32)
+    R = q_start.shape[0]
+    for t, nm in ((q_start, "q_start"), (q_len, "q_len"), (slots, "slots")):
+        _check(t, nm, (R,), torch.int32)
+    _check(row_req, "row_req", (T,), torch.int32)
+    ch, ks, wg_cols = matrix_memory_layout(d, dv, single_tokens)
+    s_off = _memory_max_floats(n_heads)
+    if s_off + n_heads * (dv + 1) * ch * ks > state.shape[1]:
+        raise KernelError("matrix_memory: the state rows are too short")
+    out = torch.empty((T, HV), dtype=out_dtype, device=rows.device)
+    scratch = torch.empty((T * n_heads * (dv + 2) + R * n_heads,), dtype=torch.float32, device=rows.device)
+    o_raw = scratch.data_ptr()
+    floor = o_raw + 4 * T * n_heads * (dv + 1)
+    m_end = floor + 4 * T * n_heads
+    _call(load_module("matrix_memory"), "ifx_matrix_memory",
+          (P, I, I, I, I, I, I, P, I, I, I, P, P, F, F, P, F, P, LL, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P),
+          rows.data_ptr(), _dt(rows), ld, q_col, k_col, v_col, g_col, gates.data_ptr(), ldg, i_col, f_col, i_bias.data_ptr(),
+          f_bias.data_ptr(), float(cap), float(d) ** -0.5, norm_weight.data_ptr(), float(eps), state.data_ptr(), state.shape[1], s_off,
+          q_start.data_ptr(), q_len.data_ptr(), slots.data_ptr(), row_req.data_ptr(), o_raw, floor, m_end, out.data_ptr(), _DT[out_dtype],
+          T, R, n_heads, d, dv, ch, ks, wg_cols, _stream())
     return out
 
 

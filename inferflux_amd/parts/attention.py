@@ -36,8 +36,12 @@ Optional mechanisms, each a constructor argument that is off by default:
                       exp(lq1 . lk1) - exp(lq2 . lk2) + c (four tensors of head_dim, one lambda for the layer), then
                       o / sqrt(mean(o^2) + e) over the head's values, times (1 - c).  Needs a position part that leaves q
                       and k alone.
+  ``sinks``           a learned score per query head ("sink" [heads]) that joins its softmax's denominator, beside or instead of
+                      the constant ``sink``; it is not scaled and has no value.
+  ``q_temp``          {"coef": c, "every": n}: the query at position p is multiplied by 1 + c ln(floor((p + 1) / n) + 1), in
+                      float, before it is rounded.
   ``tensors``         full names of the tensors in the model file ("q", "k", "v", "o", "q_bias", "k_bias", "v_bias", "gate",
-                      "mix", "q_norm", "k_norm", "lq1", "lk1", "lq2", "lk2") where they are not ``<name>.q_proj.weight`` and so on.
+                      "mix", "q_norm", "k_norm", "lq1", "lk1", "lq2", "lk2", "sink") where they are not ``<name>.q_proj.weight`` and so on.
 """
 from __future__ import annotations
 
@@ -63,7 +67,8 @@ class PagedAttention(Mixer):
                  scale: Optional[float] = None, init_std: float = 0.02, v_head_dim: Optional[int] = None,
                  keep_first: int = 0, sink: Optional[float] = None, unit_norm_eps: Optional[float] = None,
                  output_gate=False, value_mix: Optional[str] = None, tensors: Optional[Mapping[str, str]] = None,
-                 qk_norm_eps: Optional[float] = None, chunk: Optional[int] = None, differential: Optional[Mapping[str, float]] = None):
+                 qk_norm_eps: Optional[float] = None, chunk: Optional[int] = None, differential: Optional[Mapping[str, float]] = None,
+                 sinks: bool = False, q_temp: Optional[Mapping[str, float]] = None):
         """``v_head_dim``: the width of a value head where it differs from ``head_dim`` (such a layer runs on the
         kernels that take both widths: the plain attention kernel and the unfused projection path)."""
         if n_heads % n_kv_heads:
@@ -99,10 +104,20 @@ class PagedAttention(Mixer):
                       "v_bias": f"{name}.v_proj.bias", "gate": f"{name}.gate.weight", "mix": f"{name}.value_mix",
                       "q_norm": f"{name}.q_norm.weight", "k_norm": f"{name}.k_norm.weight",
                       "lq1": f"{name}.lambda_q1", "lk1": f"{name}.lambda_k1", "lq2": f"{name}.lambda_q2", "lk2": f"{name}.lambda_k2"}
+        self.names["sink"] = f"{name}.sink"
         self.names.update(tensors or {})
+        self.has_sinks, self.sinks = bool(sinks), None
+        self.q_temp = (float(q_temp["coef"]), int(q_temp["every"])) if q_temp is not None else None
+        if self.q_temp is not None and self.q_temp[1] <= 0:
+            raise ValueError(f"{name}: q_temp counts steps of {self.q_temp[1]} positions")
+        if differential is not None and (self.has_sinks or self.q_temp is not None):
+            raise ValueError(f"{name}: differential attention takes no sinks and no query temperature")
+        if self.has_sinks and self.sink is not None:
+            raise ValueError(f"{name}: a sink per head and a constant one")
         # (what the kernels fused for the plain case do not do: then the projection, the row kernel and attention run one by one)
         self._extras = (self.unit_norm_eps is not None or self.output_gate or self.value_mix is not None
-                        or self.qk_norm_eps is not None or self.chunk is not None or self.differential is not None)
+                        or self.qk_norm_eps is not None or self.chunk is not None or self.differential is not None
+                        or self.has_sinks or self.q_temp is not None)
         if self.differential is not None and (self.unit_norm_eps is not None or self.qk_norm_eps is not None
                                               or self.position.kernel_args.__func__ is not PositionEncoding.kernel_args):
             raise ValueError(f"{name}: differential attention takes no norms on q and k and a position part that leaves them alone")
@@ -141,6 +156,8 @@ class PagedAttention(Mixer):
         if self.qk_norm_eps is not None:
             out[nm["q_norm"]] = ParamSpec((d,), ("ones",))
             out[nm["k_norm"]] = ParamSpec((d,), ("ones",))
+        if self.has_sinks:
+            out[nm["sink"]] = ParamSpec((self.n_heads,), ("normal", 1.0))
         if self.differential is not None:
             for k in ("lq1", "lk1", "lq2", "lk2"):
                 out[nm[k]] = ParamSpec((self.map_dim,), ("normal", 0.1))
@@ -165,6 +182,8 @@ class PagedAttention(Mixer):
             self.q_norm_w, self.k_norm_w = tensors[nm["q_norm"]], tensors[nm["k_norm"]]
             if self.q_norm_w.dtype != self.k_norm_w.dtype:
                 self.q_norm_w, self.k_norm_w = self.q_norm_w.float(), self.k_norm_w.float()
+        if self.has_sinks:
+            self.sinks = tensors[nm["sink"]].float().contiguous()      # float whatever the file holds
         if self.differential is not None:      # one number for the layer, formed once in double precision
             dot = lambda a, b: float((tensors[nm[a]].double() * tensors[nm[b]].double()).sum().item())
             self.lam = math.exp(dot("lq1", "lk1")) - math.exp(dot("lq2", "lk2")) + self.differential[0]
@@ -192,7 +211,7 @@ class PagedAttention(Mixer):
 
     def _attend(self, q, cache, ctx, gate=None):
         if self.differential is None:
-            return paged_attention(q, cache, ctx, self.window, self.scale, self.keep_first, self.sink, gate, block=self.chunk)
+            return paged_attention(q, cache, ctx, self.window, self.scale, self.keep_first, self.sink, gate, self.sinks, block=self.chunk)
         lam, out_scale, eps = self.lam, 1.0 - self.differential[0], self.differential[1]
         if (self.v_head_dim == self.head_dim and gate is None and self.sink is None and not self.keep_first
                 and ops.mfma_attention_supported(q.dtype, self.head_dim, cache.page_size)):
@@ -209,7 +228,7 @@ class PagedAttention(Mixer):
         """The step with the optional mechanisms: the fused projection (with the gate's rows), one row kernel for bias,
         rotation, unit norms, value mixing and the cache write, attention with the gate as a factor on its output."""
         if not binding.writes_cache:
-            raise ValueError(f"{self.name}: a layer with unit norms, an output gate or value mixing owns its cache")
+            raise ValueError(f"{self.name}: a layer with unit norms, an output gate, value mixing, sinks or a query temperature owns its cache")
         cache, nH, nKV, d, dv, T = binding.cache, self.n_heads, self.n_kv_heads, self.head_dim, self.v_head_dim, h.shape[0]
         style, rotary_dim, cos, sin = self.position.kernel_args(ctx)
         if self.position.needs_apply:
@@ -229,9 +248,12 @@ class PagedAttention(Mixer):
             v_first = ctx.shared(key)
             if v_first is None:
                 raise ValueError(f"{self.name}: mixes in the values of an earlier layer, but none has handed any on in this step")
+        q_mult = None
+        if self.q_temp is not None:           # (once per step for all layers with the same constants)
+            q_mult = ctx.derived(("query_temperature", *self.q_temp), lambda: ops.query_temperature(ctx.positions, *self.q_temp))
         q = ops.rope_append(qkv, self.b_qkv, ctx.write_slots(cache.group), cos, sin, style, rotary_dim, nH, nKV, d, cache.k, cache.v,
                             cache.page_size, dv, self.unit_norm_eps, gate, v_first, self.mix_weight, v_out, qk_norm,
-                            self.gate_rows if self.gate_elementwise else 0)
+                            self.gate_rows if self.gate_elementwise else 0, q_mult)
         if t is not None:
             t.mark("mixer.qkv")
         a = self._attend(q, cache, ctx, gate)

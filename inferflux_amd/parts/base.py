@@ -24,14 +24,16 @@ Categories and what each must provide beyond ``param_specs`` / ``load``:
   injection forward(residual, ctx, embedded) -> None: changes the float32 stream in place right before the layer of the
             schedule entry that names it.  ``embedded`` is the embedding's output for the step's rows as it was before the
             first layer (kept for the step only if some injection says ``needs_embedding``).  Whatever the block before
-            has not added to the stream yet is added later as before; an addition commutes.
+            has not added to the stream yet is added later as before; an addition commutes.  A part that replaces the stream
+            overrides apply(residual, pending, ctx, embedded) -> (residual, pending) instead, which is given what is
+            pending (never rows prepared for a norm).
 
 A norm's kernel can be saved for steps of few rows, where a launch costs as much as the work.  This is
 optional for every part; one that declares nothing is run as above.
 
   norm      ``rms_params()`` -> (weight, eps) if the norm is x * rsqrt(mean(x^2) + eps) * weight, else None.
-            Such a norm's forward also takes ``SliceSums`` (a product left as partial sums; kernels/ops.py) for
-            its delta, as ``ops.add_rmsnorm`` does.
+            Such a norm's forward also takes ``SliceSums`` (a product left as partial sums; kernels/ops.py) and
+            ``DeltaSum`` (several deltas, each with a factor) for its delta, as ``ops.add_rmsnorm`` does.
   mixer,    ``adds_to_stream`` True: forward takes ``sink=StreamSink(stream, weight, eps)`` (or None) and may
   ffn       then add its result to the stream itself and return ``ScaledRows`` (the rows the norm that follows
             would give, up to a factor per row; kernels/ops.py) instead of a delta, or return its delta as
@@ -181,6 +183,10 @@ class Norm(Part):
 
 class Injection(Part):
     needs_embedding = False
+
+    def apply(self, residual: torch.Tensor, pending, ctx, embedded: Optional[torch.Tensor]):
+        self.forward(residual, ctx, embedded)
+        return residual, pending
 
     def forward(self, residual: torch.Tensor, ctx, embedded: Optional[torch.Tensor]) -> None:
         raise NotImplementedError

@@ -22,6 +22,10 @@ next sub-block (of this layer or the next) updates them first, so a sub-block co
 the model asks the block to ``close_stream``: the pending update, then the sum of the streams as the one stream that the
 final norm reads.
 
+"parallel" has one norm and hands its output to both sub-blocks: h = norm(x), x <- x + mixer(h) + ff(h) (a layer without
+feed-forward leaves the second term out).  Neither sub-block waits for the other's addition, so their outputs travel on
+together as one pending ``DeltaSum``, and the next norm adds them all in the kernel that normalises.
+
 For steps of few rows a sub-block that can do so adds its output to the stream in its last product's
 epilogue and hands on the next norm's rows up to a factor per row (``ScaledRows``), which the sub-block
 after it applies to its first product's sums: the norm between them then needs no kernel.  Parts that
@@ -32,9 +36,12 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from ..kernels.ops import ScaledDelta, ScaledRows
+from ..kernels.ops import DeltaSum, ScaledDelta, ScaledRows
 from .base import Block, MixerBinding, StreamSink, build_part, register_part
 from .plan import LayerSpec, ParamSpec
+
+
+_PARTIAL_SUMS_WELCOME = StreamSink(None, None, 0.0)
 
 
 def normed_for(norm, reader, residual, pending, ctx):
@@ -111,6 +118,67 @@ class PreNormBlock(Block):
         return residual, out
 
 
+class _BothRead:
+    """What ``normed_for`` asks on behalf of sub-blocks that read the same rows."""
+
+    def __init__(self, *parts):
+        self.parts = parts
+
+    def accepts_scaled_rows(self, n_rows: int) -> bool:
+        return all(getattr(p, "accepts_scaled_rows", None) is not None and p.accepts_scaled_rows(n_rows) for p in self.parts)
+
+
+@register_part("block", "parallel")
+class ParallelBlock(Block):
+    """Mixer and feed-forward side by side behind one norm (see the module's text).  In steps of few rows a sub-block may add
+    its output to the stream in its product's epilogue; the rows which the last of them prepares for the next norm are handed
+    on only if everything else is in the stream by then."""
+    graph_safe = True
+
+    def __init__(self, layer: LayerSpec, hidden_size: int):
+        if layer.norm_in is None or layer.norm_post is not None or layer.extra:
+            raise ValueError(f"layer {layer.prefix}: the parallel block is one norm, a mixer and optionally a feed-forward")
+        self.prefix = layer.prefix
+        self.norm_in = build_part("norm", layer.norm_in, hidden_size=hidden_size)
+        self.mixer = build_part("mixer", layer.mixer, hidden_size=hidden_size)
+        self.ffn = build_part("ffn", layer.ffn, hidden_size=hidden_size) if layer.ffn is not None else None
+        self._readers = _BothRead(*(p for p in (self.mixer, self.ffn) if p is not None))
+
+    def children(self):
+        return tuple(p for p in (self.norm_in, self.mixer, self.ffn) if p is not None)
+
+    def entry_norm(self):
+        return self.norm_in
+
+    @staticmethod
+    def _run(part, h, ctx, binding, sink):
+        if not getattr(part, "adds_to_stream", False):
+            return part.forward(h, ctx, *binding)
+        return part.forward(h, ctx, *binding, sink=sink)
+
+    def forward(self, residual, pending, ctx, binding: MixerBinding, following=None):
+        t = ctx.timer
+        params = following.rms_params() if following is not None else None
+        sink = StreamSink(residual, *params) if params is not None else _PARTIAL_SUMS_WELCOME
+        if t is not None:
+            t.enter("norm")
+        h = normed_for(self.norm_in, self._readers, residual, pending, ctx)
+        if t is not None:
+            t.mark("norm"); t.enter("mixer")
+        out = self._run(self.mixer, h, ctx, (binding,), sink)
+        if t is not None:
+            t.mark("mixer")
+        if self.ffn is None:
+            return residual, out
+        if t is not None:
+            t.enter("ffn")
+        mixed = isinstance(out, ScaledRows)                      # the mixer's output is in the stream already
+        second = self._run(self.ffn, h, ctx, (), sink if mixed else _PARTIAL_SUMS_WELCOME)
+        if t is not None:
+            t.mark("ffn")
+        return residual, second if mixed else DeltaSum.of(out, second)
+
+
 @register_part("block", "outnorm")
 class OutputNormBlock(Block):
     """x <- x + norm_in(mixer(x)); x <- x + norm_post(ffn(x)) (the second only if the layer has a feed-forward).  What
@@ -141,6 +209,8 @@ class OutputNormBlock(Block):
             if pending is not None:                       # a delta some other arrangement left: it belongs to the stream
                 if isinstance(pending, ScaledDelta):
                     residual += pending.tensor()
+                elif isinstance(pending, DeltaSum):
+                    residual += pending.tensor(residual)
                 else:
                     residual += pending.sum(torch.float32) if hasattr(pending, "parts") else pending.float()
             h = residual if ctx.act_dtype == torch.float32 else ops.cast_rows(residual, ctx.act_dtype)
@@ -193,9 +263,6 @@ class HyperPending:
 
     def __init__(self, y, mix, out):
         self.y, self.mix, self.out = y, mix, out
-
-
-_PARTIAL_SUMS_WELCOME = StreamSink(None, None, 0.0)
 
 
 @register_part("block", "hyper")

@@ -45,7 +45,7 @@ class TokenEmbedding(Part):
         saves the norm a kernel of its own where the layer's first product takes such rows."""
         params = norm.rms_params() if norm is not None else None
         if (params is not None and 0 < ctx.n_tokens <= 16 and ctx.act_dtype == torch.bfloat16
-                and params[0].dtype == torch.bfloat16):
+                and params[0].dtype in (torch.bfloat16, torch.float32)):
             return ops.embedding_scaled(ctx.token_ids, self.table, params[0], params[1], self.scale)
         return ops.embedding(ctx.token_ids, self.table, self.scale)
 

@@ -17,6 +17,9 @@ With ``router_bias`` a bias b_r joins the logits, z = W_r h + b_r (it counts for
 "softmax" with ``renormalize`` is the softmax over the chosen logits alone.  With ``shared_ff`` a further gated feed-forward
 of that inner size runs for every row and is added, times sigmoid(w_sg . h) (one number per row) with ``shared_gate``.
 
+With ``weigh_input`` the weights multiply the experts' inputs instead of their outputs: out = sum of expert_e(w_e h) (applied,
+in float, to the sums of the gate and up products before the activation).
+
 Tensors (``<name>.``): router [experts + identity, H] (router.b [experts], correction [experts + identity]), e<j>.gate and e<j>.up [ff, H], e<j>.down [H, ff]; shared.gate,
 shared.up, shared.down, shared.sg [1, H]; no other biases.  The experts' matrices are stacked at load into [experts, ff, H]
 and [experts, H, ff].
@@ -49,7 +52,7 @@ class MixtureOfExperts(FeedForward):
                  group_top: int = 2, scoring: str = "sigmoid", renormalize: bool = False, route_scale: float = 1.0,
                  init_std: float = 0.02, router_bias: bool = False, shared_ff: int = 0, shared_gate: bool = False,
                  n_identity: int = 0, choice_bias: bool = False, activation: str = "silu", limit: Optional[float] = None,
-                 shared_limit: Optional[float] = None):
+                 shared_limit: Optional[float] = None, weigh_input: bool = False):
         if scoring not in ("sigmoid", "softmax"):
             raise ValueError(f"{name}: scoring '{scoring}' unknown (sigmoid or softmax)")
         self.n_identity = int(n_identity or 0)
@@ -65,6 +68,7 @@ class MixtureOfExperts(FeedForward):
         if (self.act == ops.ACT_CLAMPED_SWISH) != (self.limit > 0):
             raise ValueError(f"{name}: the activation '{activation}' and a limit of {limit} do not go together")
         self.choice_bias, self.correction = bool(choice_bias), None
+        self.weigh_input = bool(weigh_input)
         self.name, self.hidden_size = name, int(hidden_size)
         self.n_experts, self.top, self.ff = int(n_experts), int(top), int(ff)
         self.groups, self.keep_groups, self.group_top = int(groups), int(keep_groups), int(group_top)
@@ -135,7 +139,7 @@ class MixtureOfExperts(FeedForward):
             ctx.timer.mark("ffn.route")
         if self.up is None and x.shape[0] * self.top >= GROUPED_MIN_ITEMS:
             return self._with_shared(ops.moe_experts_grouped(x, self.gate, self.down, ids, weights, self.act, self.limit,
-                                                             self.n_identity), x, ctx)      # (partial sums, one per choice)
+                                                             self.n_identity, self.weigh_input), x, ctx)      # (partial sums, one per choice)
         out = self._with_shared(ops.moe_experts(x, self.gate, self.up, self.down, ids, weights, self.act, self.limit,
-                                                self.n_identity), x, ctx)
+                                                self.n_identity, self.weigh_input), x, ctx)
         return out if out.dtype == h.dtype else out.to(h.dtype)

@@ -9,7 +9,9 @@ Layer norm with a weight and no bias: y = (x - mean) / sqrt(var + eps) * w, var 
 deviations from the mean, all in float.  Besides the common ``forward`` it can sit on a sub-block's output
 (``add_to``: stream += norm(delta)), which is how the "outnorm" block uses it.
 
-``tensor`` names a norm's weight in full where a model file does not call it ``<name>.weight``.
+``tensor`` names a norm's weight in full where a model file does not call it ``<name>.weight``.  ``offset``: the file stores
+the weight less this number (a weight stored around zero: 1); the sum is formed in float at load and stays float, so that
+nothing of a small difference from one is rounded away.
 """
 from __future__ import annotations
 
@@ -26,16 +28,16 @@ from .plan import ParamSpec
 class RMSNorm(Norm):
     graph_safe = True
 
-    def __init__(self, name: str, hidden_size: int, eps: float, tensor: Optional[str] = None):
+    def __init__(self, name: str, hidden_size: int, eps: float, tensor: Optional[str] = None, offset: float = 0.0):
         self.name, self.hidden_size, self.eps = name, int(hidden_size), float(eps)
-        self.tensor = tensor or f"{name}.weight"
+        self.tensor, self.offset = tensor or f"{name}.weight", float(offset)
         self.weight: Optional[torch.Tensor] = None
 
     def param_specs(self) -> Dict[str, ParamSpec]:
-        return {self.tensor: ParamSpec((self.hidden_size,), ("ones",))}
+        return {self.tensor: ParamSpec((self.hidden_size,), ("zeros",) if self.offset == 1.0 else ("ones",))}
 
     def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
-        self.weight = tensors[self.tensor]
+        self.weight = tensors[self.tensor] if self.offset == 0.0 else (tensors[self.tensor].float() + self.offset).contiguous()
 
     def rms_params(self):
         return self.weight, self.eps
