@@ -169,6 +169,44 @@ VAVADRA_SIZES = {
     "medium-wide-latent-looped": (_vavadra_shape(2048, 8, 16, 2, 128, 2048, 16, 64, 128, 512, 64, (32, 4, 1408, 1408, 4), "lald", loop=(2, 6, 2)),
                                   _vavadra_twin(2048, 8, 16, 2, 128, 2048, 16, 64, 128, 128, (32, 4, 1408, 1408), "aaag")),
 }
+# Layer sizes for the comparison of the Narasun design (matrix memory with exponential gates; attention with a sink per head
+# and a query temperature beside time mixing in one layer; one norm for mixer and feed-forward; experts weighed at their
+# input; a looped span whose passes project the stream) with the framework's closest model, the Tabatar design on one stream, at
+# equal width, depth, heads, keys in sight, feed-forward work and order: its gated linear attention (the matrix state with the
+# same head sizes) stands beside the matrix memory and its attention layers beside the two mixers side by side, which hold
+# a recurrence more.  ``pattern``: "m" matrix memory, "p" the two mixers.
+def _narasun_shape(width, layers, heads, kv_heads, dim, m_heads, m_dim, m_vdim, t_heads, t_dim, rank, pattern, ff=0, moe=None, loop=None, vocab=32000):
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "q_temp": {"coef": 0.1, "every": 1024}}
+    par = {"left": att, "right": {"heads": t_heads, "dim": t_dim, "rank": rank}, "left_scale": 0.7, "right_scale": 0.7}
+    mem = {"heads": m_heads, "dim": m_dim, "vdim": m_vdim, "gate_cap": 15.0}
+    mix = {"m": ("mlstm", mem), "p": ("parallel", par)}
+    mlp = {"kind": "dense", "ff": ff} if moe is None else {"kind": "moe", "expert": {"ff": moe[2]}, "router": {"experts": moe[0], "top": moe[1]}}
+    out = {"architecture": "Narasun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+           "layers": [{"type": mix[pattern[i % len(pattern)]][0], "mixer": mix[pattern[i % len(pattern)]][1], "mlp": mlp} for i in range(layers)]}
+    if loop:
+        out["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return out
+
+
+def _narasun_twin(width, layers, heads, kv_heads, dim, g_heads, g_dim, g_vdim, rank, pattern, ff=0, moe=None):
+    return _tabatar_shape(width, layers, heads, kv_heads, dim, 8192, ff * 3 // 2, g_heads, g_dim, g_vdim, rank, pattern,
+                          moe=(*moe, 0) if moe else None, streams=None, moe_every=1)
+
+
+_NARASUN_SMALL, _NARASUN_MEDIUM = (1024, 8, 8, 2, 128, 8, 64, 128), (2048, 8, 16, 2, 128, 16, 64, 128)
+NARASUN_SIZES = {
+    "small": (_narasun_shape(*_NARASUN_SMALL, 8, 64, 64, "mmpm", moe=(16, 2, 1408)), _narasun_twin(*_NARASUN_SMALL, 64, "ggag", moe=(16, 2, 1408))),
+    "medium": (_narasun_shape(*_NARASUN_MEDIUM, 16, 64, 128, "mmpm", moe=(32, 4, 1408)), _narasun_twin(*_NARASUN_MEDIUM, 128, "ggag", moe=(32, 4, 1408))),
+    "medium-dense": (_narasun_shape(*_NARASUN_MEDIUM, 16, 64, 128, "mmpm", ff=5632), _narasun_twin(*_NARASUN_MEDIUM, 128, "ggag", ff=5632)),
+    "medium-memory": (_narasun_shape(*_NARASUN_MEDIUM, 16, 64, 128, "m", ff=5632), _narasun_twin(*_NARASUN_MEDIUM, 128, "g", ff=5632)),
+    "medium-parallel": (_narasun_shape(*_NARASUN_MEDIUM, 16, 64, 128, "p", ff=5632), _narasun_twin(*_NARASUN_MEDIUM, 128, "a", ff=5632)),
+    # heads as large models of this kind have them: 256 key channels and 512 values (the twin's heads 4 times as many, 64 x 128)
+    "medium-large-heads": (_narasun_shape(2048, 8, 16, 2, 128, 4, 256, 512, 16, 64, 128, "m", ff=5632),
+                           _narasun_twin(2048, 8, 16, 2, 128, 16, 64, 128, 128, "g", ff=5632)),
+    # layers 2 .. 5 twice: 12 layer runs
+    "medium-looped": (_narasun_shape(*_NARASUN_MEDIUM, 16, 64, 128, "mmpm", moe=(32, 4, 1408), loop=(2, 6, 2)),
+                      _narasun_twin(*_NARASUN_MEDIUM, 128, "ggag", moe=(32, 4, 1408))),
+}
 CONTEXT = 4096
 PROMPT = 2048
 DECODE_KV_START = 3072      # mean context of a 2,048-token decode after a 2,048-token prompt
@@ -192,16 +230,16 @@ def main() -> int:
     ap.add_argument("--dtype", choices=["bf16", "fp32"], default="bf16")
     ap.add_argument("--no-points", action="store_true", help="skip the batch 1 / 64 and prefill measurements")
     ap.add_argument("--no-gemm-tuning", action="store_true", help="leave the library's default kernel choice for large products")
-    ap.add_argument("--workload", choices=["decode", "prefill", "mumusun", "podurax", "tabatar", "vavadra", *WORKLOADS], default="decode",
+    ap.add_argument("--workload", choices=["decode", "prefill", "mumusun", "podurax", "tabatar", "vavadra", "narasun", *WORKLOADS], default="decode",
                     help="decode: the headline measurement; prefill: only the 2,048-token prefill, --steps times "
                          "(for profiles); mixed3b / long14b: whole workloads through the scheduler; mumusun: prefill and "
                          "decode of the Mumusun design beside the dense decoder at equal size (--size, --only-design); podurax: the same "
                          "for the Podurax design; tabatar: the Tabatar design beside the Podurax design at equal size; vavadra: the "
-                         "Vavadra design beside the Tabatar design (on one stream) at equal size")
-    ap.add_argument("--size", choices=["all", *dict.fromkeys([*DESIGN_SIZES, *PODURAX_SIZES, *TABATAR_SIZES, *VAVADRA_SIZES])], default="all",
-                    help="--workload mumusun / podurax / tabatar / vavadra: which of its sizes")
-    ap.add_argument("--only-design", choices=["both", "mumusun", "podurax", "tabatar", "vavadra", "dense"], default="both",
-                    help="--workload mumusun / podurax / tabatar / vavadra: which of the two models")
+                         "Vavadra design beside the Tabatar design (on one stream) at equal size; narasun: the Narasun design beside it")
+    ap.add_argument("--size", choices=["all", *dict.fromkeys([*DESIGN_SIZES, *PODURAX_SIZES, *TABATAR_SIZES, *VAVADRA_SIZES, *NARASUN_SIZES])], default="all",
+                    help="--workload mumusun / podurax / tabatar / vavadra / narasun: which of its sizes")
+    ap.add_argument("--only-design", choices=["both", "mumusun", "podurax", "tabatar", "vavadra", "narasun", "dense"], default="both",
+                    help="--workload mumusun / podurax / tabatar / vavadra / narasun: which of the two models")
     ap.add_argument("--no-decode-weight-copy", action="store_true",
                     help="decode from the weights' plain rows instead of the tiled copy")
     ap.add_argument("--ceilings", action=argparse.BooleanOptionalAction, default=True,
@@ -244,6 +282,8 @@ def main() -> int:
         return run_design_compare(args, TABATAR_SIZES, "tabatar", twin="podurax")
     if args.workload == "vavadra":
         return run_design_compare(args, VAVADRA_SIZES, "vavadra", twin="tabatar")
+    if args.workload == "narasun":
+        return run_design_compare(args, NARASUN_SIZES, "narasun", twin="tabatar")
     if args.workload == "mumusun":
         return run_design_compare(args)
     shape = dict({"7b": SHAPE_7B, "3b": SHAPE_3B, "14b": SHAPE_14B, "1.5b": SHAPE_15B, "0.5b": SHAPE_05B, "32b": SHAPE_32B,

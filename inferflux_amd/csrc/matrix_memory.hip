@@ -15,11 +15,21 @@
 // m [H, padded to a multiple of 4], then S laid out [head][column 0 .. dv][d_pad], d_pad = CH * KS >= d (padding stays zero).
 // The columns of S never meet, so a head's columns are dealt to several workgroups of ``cols`` columns each.  In a workgroup
 // thread (column, run) holds CH consecutive key channels of its column in registers; the KS threads of a column are
-// neighbouring lanes and add their parts of S^T q in a fixed order.  Tokens are taken STAGE at a time: all threads load the
+// neighbouring lanes and add their parts of S^T q in a fixed order.  Tokens are taken a stage of STAGE (fewer for wide heads) at a time: all threads load the
 // stage's q, k and their columns of v into LDS, one wave forms the gates and the running maximum of the stage (the maximum
 // as a scan over its lanes: m after a token is max(m + F, M) of the composed pairs (F, M)), everybody walks the tokens.  Read-outs
-// go to ``o_raw`` [T, H, dv + 1] (float); a second kernel, a wave per (token, head), divides, norms and gates them, and
-// writes a request's last m into its state (the walk's workgroups all read the old one).
+// go to ``o_raw`` [T, H, dv] and, of the normaliser's column, ``nq`` [T, H] (float); a second kernel, a wave per (token, head),
+// divides, norms and gates them, and writes a request's last m into its state (the walk's workgroups all read the old one).
+//
+// Long portions in bfloat16 are cut into chunks of 64 tokens that run side by side on the matrix cores.  With F the sum of f
+// from a chunk's start and m0 the maximum before the chunk, for tokens s <= t of a chunk
+//   o_t = exp(F_t + m0 - m_t) S0^T q_t + sum_s exp(F_t - F_s + i_s - m_t) (q_t . k_s) v_s          (every exponent is <= 0)
+//   S_end = exp(F_L + m0 - m_L) S0 + sum_s exp(F_L - F_s + i_s - m_L) k_s v_s^T
+// in four launches: the gates and maxima of all tokens (a wave per request and head, exact for the whole portion, so nothing is
+// ever rescaled), each chunk's own sum of outer products, the walk over a request's chunks that leaves S0 of every chunk, and
+// the read-outs.  q, k and v are the projections' bfloat16 numbers as they are; what is float on the way into a product (S0,
+// the weighted keys, the weighted scores) goes in as two bfloat16 numbers, the rounded one and the rest, so that nothing of
+// the recurrence is rounded to 16 bits.  The normaliser's sums are plain float.
 #include "common.h"
 #include "lane_sums.h"
 
@@ -34,11 +44,12 @@ struct MemoryArgs {
   const float* norm_w; float eps;              // [H dv]
   float* state; size_t state_stride; int s_off;
   const int* q_start; const int* q_len; const int* slots; const int* row_req;
-  float* o_raw;        // [T, H, dv + 1]
+  float* o_raw;        // [T, H, dv]
+  float* nq;           // [T, H]: n . q * q_scale
   float* floor;        // [T, H]: exp(-m_t)
-  float* m_end;        // [R, H]
+  float* m_end;        // [R, H], or null: the state's maxima are up to date
   void* out;           // [T, H dv]
-  int T, R, H, d, dv, KS, cols;
+  int T, R, H, d, dv, KS, cols, stage;      // stage: tokens taken at a time (at most STAGE)
 };
 
 __device__ __forceinline__ float log_sigmoid(float x) {      // -softplus(-x), without overflow
@@ -56,9 +67,10 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(MemoryArgs a) {
   if (n <= 0) return;
   const int t0 = a.q_start[r], d = a.d, KS = a.KS, dpad = CH * KS;
   const int cols = min(a.cols, n_cols - j0);
+  const int stage = a.stage;
   float* q_s = lds;
-  float* k_s = lds + STAGE * dpad;
-  float* v_s = lds + 2 * STAGE * dpad;
+  float* k_s = lds + stage * dpad;
+  float* v_s = lds + 2 * stage * dpad;
   const int tid = threadIdx.x, nthr = blockDim.x, lane = tid % WAVE;
   const int jl = tid / KS, s = tid % KS;
   const bool owner = jl < cols;
@@ -75,8 +87,8 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(MemoryArgs a) {
   const TI* rows = (const TI*)a.rows;
   const LaneSteps steps = lane_steps(KS);
   const int dshift = __ffs(dpad) - 1;
-  for (int base = 0; base < n; base += STAGE) {
-    const int cnt = min(STAGE, n - base);
+  for (int base = 0; base < n; base += stage) {
+    const int cnt = min(stage, n - base);
     if (tid < WAVE) {
       // the stage's gates, a token a lane, and the running maximum as a scan of the pairs (F: sum of f, M: the best exponent)
       const bool in = lane < cnt;
@@ -122,7 +134,11 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(MemoryArgs a) {
           o4[c & 3] = fmaf(S[c], qp[c], o4[c & 3]);
         }
         const float o = column_sum((o4[0] + o4[1]) + (o4[2] + o4[3]), steps);
-        if (s == 0) a.o_raw[((size_t)(t0 + base + tt) * a.H + h) * n_cols + j0 + jl] = o;
+        const size_t item = (size_t)(t0 + base + tt) * a.H + h;
+        if (s == 0) {
+          if (j0 + jl < a.dv) a.o_raw[item * a.dv + j0 + jl] = o;
+          else a.nq[item] = o;
+        }
       }
     }
     __syncthreads();
@@ -142,8 +158,8 @@ __global__ __launch_bounds__(256) void memory_finish_kernel(MemoryArgs a) {
   if (item >= (size_t)a.T * a.H) return;
   const size_t t = item / a.H;
   const int h = (int)(item % a.H), dv = a.dv;
-  const float* o = a.o_raw + item * (dv + 1);
-  const float inv_den = 1.0f / (fmaxf(fabsf(o[dv]), a.floor[item]) + 1e-6f);
+  const float* o = a.o_raw + item * dv;
+  const float inv_den = 1.0f / (fmaxf(fabsf(a.nq[item]), a.floor[item]) + 1e-6f);
   float ss = 0.f;
   for (int c = lane; c < dv; c += WAVE) { const float v = o[c] * inv_den; ss = fmaf(v, v, ss); }
   const float f = inv_den / sqrtf(wave_sum(ss) / (float)dv + a.eps);
@@ -152,31 +168,360 @@ __global__ __launch_bounds__(256) void memory_finish_kernel(MemoryArgs a) {
     const float g = to_f(rows[t * a.ld + a.g_col + (size_t)h * dv + c]);
     ((TO*)a.out)[item * dv + c] = from_f<TO>(o[c] * f * a.norm_w[(size_t)h * dv + c] / (1.0f + expf(-g)));
   }
+  if (!a.m_end) return;
   const int r = a.row_req[t];
   if (lane == 0 && (int)t == a.q_start[r] + a.q_len[r] - 1)
     a.state[(size_t)a.slots[r] * a.state_stride + h] = a.m_end[(size_t)r * a.H + h];
 }
 
+// ---------------------------------------------------------------------------------------
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
+typedef __attribute__((__vector_size__(4 * sizeof(__bf16)))) __bf16 bf16x4;
+typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
+typedef __attribute__((__vector_size__(16 * sizeof(float)))) float floatx16;
+
+#define CL 64                // tokens of a chunk
+#define CJ 128               // value columns of a workgroup
+#define CI 64                // key channels of a workgroup of the chunks' sums
+#define CLP (CL + 8)         // a row of 64 tokens in LDS, padded against bank conflicts
+
+struct ChunkArgs {
+  MemoryArgs a;
+  const int* chunk_req; const int* chunk_t0; const int* chunk_len; const int* req_chunk0;
+  float* cum_f; float* log_i; float* m;        // [H, T]: sum of f from the token's chunk's start, i, the maximum after the token
+  float* m0;           // [n_chunks, H]: the maximum before the chunk
+  float* keep;         // [n_chunks, H]: exp(F_L + m0 - m_L)
+  float* chunk_state;  // [n_chunks, H, dv + 1, dpad]
+  int n_chunks, dpad;
+};
+
+__device__ __forceinline__ bf16x8 zero8() {
+  bf16x8 z;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) z[i] = (__bf16)0.f;
+  return z;
+}
+
+// A wave per (request, head): a chunk's tokens a lane each.
+__global__ __launch_bounds__(WAVE) void memory_gates_kernel(ChunkArgs c) {
+  const MemoryArgs& a = c.a;
+  const int h = blockIdx.x, r = blockIdx.y, lane = threadIdx.x;
+  const int n = a.q_len[r];
+  if (n <= 0) return;
+  const int t0 = a.q_start[r], c0 = c.req_chunk0[r];
+  float* m_state = a.state + (size_t)a.slots[r] * a.state_stride + h;
+  float m = *m_state;
+  const float ib = a.i_bias[h], fb = a.f_bias[h];
+  float gi = 0.f, gf = 0.f;
+  auto fetch = [&](int base) {
+    if (base + lane < n) {
+      const float* g = a.gates + (size_t)(t0 + base + lane) * a.ldg;
+      gi = g[a.i_col + h]; gf = g[a.f_col + h];
+    }
+  };
+  fetch(0);
+  for (int base = 0, k = 0; base < n; base += CL, ++k) {
+    const int cnt = min(CL, n - base);
+    const bool in = lane < cnt;
+    const float li = in ? soft_cap(gi + ib, a.cap) : -INFINITY;
+    const float lf = in ? log_sigmoid(soft_cap(gf + fb, a.cap)) : 0.f;
+    fetch(base + CL);                  // the next chunk's are on their way during the scan
+    float F = lf, M = li;
+#pragma unroll
+    for (int o = 1; o < CL; o <<= 1) {
+      const float Fp = __shfl_up(F, o, WAVE), Mp = __shfl_up(M, o, WAVE);
+      if (lane >= o) { M = fmaxf(Mp + F, M); F += Fp; }
+    }
+    const float mt = fmaxf(m + F, M);
+    if (in) {
+      const size_t at = (size_t)h * a.T + t0 + base + lane;
+      c.cum_f[at] = F; c.log_i[at] = li; c.m[at] = mt;
+      a.floor[(size_t)(t0 + base + lane) * a.H + h] = expf(-mt);
+    }
+    const float m_last = __shfl(mt, cnt - 1, WAVE), F_last = __shfl(F, cnt - 1, WAVE);
+    if (lane == 0) {
+      c.m0[(size_t)(c0 + k) * a.H + h] = m;
+      c.keep[(size_t)(c0 + k) * a.H + h] = expf(F_last + m - m_last);
+    }
+    m = m_last;
+  }
+  if (lane == 0) *m_state = m;
+}
+
+// value columns j0 .. of head h's v, tokens in pairs, as rows [column][token] of LDS (zeros beyond dv and beyond the chunk)
+__device__ __forceinline__ void stage_columns(const MemoryArgs& a, int col, int width, int w0, int n_cols, int t0, int len, bf16_t (*dst)[CLP]) {
+  const bf16_t* rows = (const bf16_t*)a.rows;
+  for (int x = threadIdx.x; x < (CL / 2) * (n_cols / 8); x += 256) {
+    const int p = x % (CL / 2), g = x / (CL / 2), s = 2 * p, w = w0 + 8 * g;
+    const bf16_t* src = rows + (size_t)(t0 + s) * a.ld + col + w;
+    const bf16x8 u = (s < len && w < width) ? *(const bf16x8*)src : zero8();
+    const bf16x8 v = (s + 1 < len && w < width) ? *(const bf16x8*)(src + a.ld) : zero8();
+#pragma unroll
+    for (int e = 0; e < 8; ++e) *(bf16x2*)&dst[8 * g + e][s] = bf16x2{u[e], v[e]};
+  }
+}
+
+// A chunk's own sum: chunk_state[chunk][h][j][i] = sum_s w_s k_s[i] v_s[j], w_s = exp(F_L - F_s + i_s - m_L), for CJ columns and CI
+// channels; the workgroups of the first columns form the normaliser's column too.
+__global__ __launch_bounds__(256) void memory_chunk_sums_kernel(ChunkArgs c) {
+  const MemoryArgs& a = c.a;
+  __shared__ __attribute__((aligned(16))) bf16_t vt[CJ][CLP];
+  __shared__ __attribute__((aligned(16))) bf16_t kh[CI][CLP];
+  __shared__ __attribute__((aligned(16))) bf16_t kl[CI][CLP];
+  __shared__ float wt[CL];
+  const int n_jb = (a.dv + CJ - 1) / CJ;
+  const int chunk = blockIdx.x, h = blockIdx.y, j0 = (blockIdx.z % n_jb) * CJ, i0 = (blockIdx.z / n_jb) * CI;
+  const int t0 = c.chunk_t0[chunk], len = c.chunk_len[chunk], tid = threadIdx.x;
+  if (tid < CL) {
+    const float* F = c.cum_f + (size_t)h * a.T + t0;
+    wt[tid] = tid < len ? expf(F[len - 1] - F[tid] + c.log_i[(size_t)h * a.T + t0 + tid] - c.m[(size_t)h * a.T + t0 + len - 1]) : 0.f;
+  }
+  stage_columns(a, a.v_col + h * a.dv, a.dv, j0, CJ, t0, len, vt);
+  __syncthreads();
+  const bf16_t* rows = (const bf16_t*)a.rows;
+  for (int x = tid; x < (CL / 2) * (CI / 8); x += 256) {        // the keys, weighted, in two parts each
+    const int p = x % (CL / 2), g = x / (CL / 2), s = 2 * p, i = i0 + 8 * g;
+    const bf16_t* src = rows + (size_t)(t0 + s) * a.ld + a.k_col + h * a.d + i;
+    const bf16x8 u = (s < len && i < a.d) ? *(const bf16x8*)src : zero8();
+    const bf16x8 v = (s + 1 < len && i < a.d) ? *(const bf16x8*)(src + a.ld) : zero8();
+    const float w0 = wt[s], w1 = wt[s + 1];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float x0 = (float)u[e] * w0, x1 = (float)v[e] * w1;
+      const bf16x2 hi = bf16x2{(__bf16)x0, (__bf16)x1};
+      *(bf16x2*)&kh[8 * g + e][s] = hi;
+      *(bf16x2*)&kl[8 * g + e][s] = bf16x2{(__bf16)(x0 - (float)hi[0]), (__bf16)(x1 - (float)hi[1])};
+    }
+  }
+  __syncthreads();
+  float* out = c.chunk_state + ((size_t)chunk * a.H + h) * (a.dv + 1) * c.dpad;
+  if (j0 == 0 && tid < CI && i0 + tid < c.dpad) {
+    float n = 0.f;
+    for (int s = 0; s < CL; ++s) n += (float)kh[tid][s] + (float)kl[tid][s];
+    out[(size_t)a.dv * c.dpad + i0 + tid] = n;
+  }
+  const int wave = tid / WAVE, lane = tid % WAVE, l32 = lane & 31, hi = lane >> 5;
+  const int j = j0 + 32 * wave + l32;
+  if (j0 + 32 * wave >= a.dv) return;
+  floatx16 acc[CI / 32];
+#pragma unroll
+  for (int it = 0; it < CI / 32; ++it)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) acc[it][e] = 0.f;
+#pragma unroll
+  for (int ks = 0; ks < CL / 16; ++ks) {
+    const bf16x8 b = *(const bf16x8*)&vt[32 * wave + l32][16 * ks + 8 * hi];
+#pragma unroll
+    for (int it = 0; it < CI / 32; ++it) {
+      const bf16x8 ah = *(const bf16x8*)&kh[32 * it + l32][16 * ks + 8 * hi], al = *(const bf16x8*)&kl[32 * it + l32][16 * ks + 8 * hi];
+      acc[it] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(ah, b, acc[it], 0, 0, 0);
+      acc[it] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(al, b, acc[it], 0, 0, 0);
+    }
+  }
+  if (j >= a.dv) return;
+#pragma unroll
+  for (int it = 0; it < CI / 32; ++it)
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int i = i0 + 32 * it + 8 * q + 4 * hi;
+      if (i < c.dpad) *(float4*)(out + (size_t)j * c.dpad + i) = make_float4(acc[it][4 * q], acc[it][4 * q + 1], acc[it][4 * q + 2], acc[it][4 * q + 3]);
+    }
+}
+
+// Four numbers of a request's S a thread: walks the request's chunks; a chunk's own sum becomes the S it starts from.
+#define WALK_AHEAD 8
+__global__ __launch_bounds__(256) void memory_combine_kernel(ChunkArgs c) {
+  const MemoryArgs& a = c.a;
+  const size_t per = (size_t)a.H * (a.dv + 1) * c.dpad;
+  const size_t e = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
+  if (e >= per) return;
+  const int r = blockIdx.y, c0 = c.req_chunk0[r], c1 = c.req_chunk0[r + 1];
+  if (c1 <= c0) return;
+  const int h = (int)(e / ((size_t)(a.dv + 1) * c.dpad));
+  float4* slot = (float4*)(a.state + (size_t)a.slots[r] * a.state_stride + a.s_off + e);
+  float4 S = *slot;
+  for (int k0 = c0; k0 < c1; k0 += WALK_AHEAD) {
+    float4 mine[WALK_AHEAD];
+    float keep[WALK_AHEAD];
+#pragma unroll
+    for (int u = 0; u < WALK_AHEAD; ++u) {
+      const int k = min(k0 + u, c1 - 1);
+      mine[u] = *(const float4*)(c.chunk_state + (size_t)k * per + e);
+      keep[u] = c.keep[(size_t)k * a.H + h];
+    }
+#pragma unroll
+    for (int u = 0; u < WALK_AHEAD; ++u) {
+      if (k0 + u >= c1) break;
+      *(float4*)(c.chunk_state + (size_t)(k0 + u) * per + e) = S;
+      S.x = fmaf(keep[u], S.x, mine[u].x); S.y = fmaf(keep[u], S.y, mine[u].y);
+      S.z = fmaf(keep[u], S.z, mine[u].z); S.w = fmaf(keep[u], S.w, mine[u].w);
+    }
+  }
+  *slot = S;
+}
+
+// The read-outs of a chunk's tokens for CJ columns of a head.
+__global__ __launch_bounds__(256) void memory_chunk_out_kernel(ChunkArgs c) {
+  const MemoryArgs& a = c.a;
+  __shared__ __attribute__((aligned(16))) bf16_t vt[CJ][CLP];
+  __shared__ __attribute__((aligned(16))) bf16_t ph[CL][CLP];
+  __shared__ __attribute__((aligned(16))) bf16_t pl[CL][CLP];
+  __shared__ float Fs[CL], is[CL], ms[CL], row_sum[2][CL];
+  const int chunk = blockIdx.x, h = blockIdx.y, j0 = blockIdx.z * CJ;
+  const int t0 = c.chunk_t0[chunk], len = c.chunk_len[chunk], tid = threadIdx.x, d = a.d;
+  const int wave = tid / WAVE, lane = tid % WAVE, l32 = lane & 31, hi = lane >> 5;
+  const bf16_t* rows = (const bf16_t*)a.rows;
+  const bf16_t* qb = rows + (size_t)t0 * a.ld + a.q_col + h * d;
+  const bf16_t* kb = rows + (size_t)t0 * a.ld + a.k_col + h * d;
+  const float m0 = c.m0[(size_t)chunk * a.H + h];
+  if (tid < CL) {
+    const size_t at = (size_t)h * a.T + t0 + min(tid, len - 1);
+    Fs[tid] = c.cum_f[at]; is[tid] = c.log_i[at]; ms[tid] = c.m[at];
+  }
+  stage_columns(a, a.v_col + h * a.dv, a.dv, j0, CJ, t0, len, vt);
+  auto load_row = [&](const bf16_t* base, int row, int k) { return (row < len && k < d) ? *(const bf16x8*)(base + (size_t)row * a.ld + k) : zero8(); };
+  // scores, transposed: wave (wt, ws) forms the 32 keys 32 ws ... against the 32 queries 32 wt ...
+  const int wt = wave & 1, ws = wave >> 1;
+  floatx16 sc;
+#pragma unroll
+  for (int e = 0; e < 16; ++e) sc[e] = 0.f;
+  if (ws <= wt)          // (keys behind all of the tile's queries weigh nothing)
+    for (int k = 8 * hi; k < d + 8 * hi; k += 16) {
+      const bf16x8 kk = load_row(kb, 32 * ws + l32, k), qq = load_row(qb, 32 * wt + l32, k);
+      sc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kk, qq, sc, 0, 0, 0);
+    }
+  __syncthreads();
+  {
+    const int t = 32 * wt + l32;
+    const float Ft = Fs[t], mt = ms[t];
+    float sum = 0.f;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      bf16x4 yh, yl;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int s = 32 * ws + 8 * q + 4 * hi + e;
+        const float p = (s <= t && t < len) ? sc[4 * q + e] * a.q_scale * expf(Ft - Fs[s] + is[s] - mt) : 0.f;
+        sum += p;
+        yh[e] = (__bf16)p;
+        yl[e] = (__bf16)(p - (float)yh[e]);
+      }
+      *(bf16x4*)&ph[t][32 * ws + 8 * q + 4 * hi] = yh;
+      *(bf16x4*)&pl[t][32 * ws + 8 * q + 4 * hi] = yl;
+    }
+    sum += __shfl_xor(sum, 32, WAVE);
+    if (hi == 0) row_sum[ws][t] = sum;
+  }
+  __syncthreads();
+  const float* S0 = c.chunk_state + ((size_t)chunk * a.H + h) * (a.dv + 1) * c.dpad;
+  if (blockIdx.z == 0) {          // the normaliser: four threads a token
+    const int t = tid >> 2, part = tid & 3;
+    float nq = 0.f;
+    if (t < len)
+      for (int i = part; i < d; i += 4) nq = fmaf((float)qb[(size_t)t * a.ld + i], S0[(size_t)a.dv * c.dpad + i], nq);
+    nq += __shfl_xor(nq, 1, WAVE);
+    nq += __shfl_xor(nq, 2, WAVE);
+    if (part == 0 && t < len)
+      a.nq[(size_t)(t0 + t) * a.H + h] = nq * a.q_scale * expf(Fs[t] + m0 - ms[t]) + row_sum[0][t] + row_sum[1][t];
+  }
+  const int j = j0 + 32 * wave + l32;
+  if (j0 + 32 * wave >= a.dv) return;
+  floatx16 acc[2];
+#pragma unroll
+  for (int tt = 0; tt < 2; ++tt)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) acc[tt][e] = 0.f;
+  // what the chunk starts from: S0's rows are asked for as floats and go in as two bfloat16 numbers
+  const float* Srow = S0 + (size_t)min(j, a.dv - 1) * c.dpad;
+  for (int k = 8 * hi; k < d + 8 * hi; k += 16) {
+    bf16x8 sh = zero8(), sl = zero8();
+    if (k < d) {
+      const float4 x = *(const float4*)(Srow + k), y = *(const float4*)(Srow + k + 4);
+      const float f[8] = {x.x, x.y, x.z, x.w, y.x, y.y, y.z, y.w};
+#pragma unroll
+      for (int e = 0; e < 8; ++e) { sh[e] = (__bf16)f[e]; sl[e] = (__bf16)(f[e] - (float)sh[e]); }
+    }
+#pragma unroll
+    for (int tt = 0; tt < 2; ++tt) {
+      const bf16x8 qq = load_row(qb, 32 * tt + l32, k);
+      acc[tt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sh, qq, acc[tt], 0, 0, 0);
+      acc[tt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sl, qq, acc[tt], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int tt = 0; tt < 2; ++tt) {
+    const int t = 32 * tt + l32;
+    const float f = a.q_scale * expf(Fs[t] + m0 - ms[t]);
+#pragma unroll
+    for (int e = 0; e < 16; ++e) acc[tt][e] *= f;
+  }
+#pragma unroll
+  for (int ks = 0; ks < CL / 16; ++ks) {
+    const bf16x8 v = *(const bf16x8*)&vt[32 * wave + l32][16 * ks + 8 * hi];
+#pragma unroll
+    for (int tt = 0; tt < 2; ++tt) {
+      if (16 * ks >= 32 * (tt + 1)) continue;        // (keys behind all of the tile's queries)
+      const bf16x8 bh = *(const bf16x8*)&ph[32 * tt + l32][16 * ks + 8 * hi], bl = *(const bf16x8*)&pl[32 * tt + l32][16 * ks + 8 * hi];
+      acc[tt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v, bh, acc[tt], 0, 0, 0);
+      acc[tt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(v, bl, acc[tt], 0, 0, 0);
+    }
+  }
+  // acc[tt][e]: column j0 + 32 wave + 8 (e / 4) + 4 hi + e % 4 of token 32 tt + l32 (dv is a multiple of 8: runs of four are whole)
+#pragma unroll
+  for (int tt = 0; tt < 2; ++tt) {
+    const int t = 32 * tt + l32;
+    if (t >= len) continue;
+    float* o = a.o_raw + ((size_t)(t0 + t) * a.H + h) * a.dv;
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int jj = j0 + 32 * wave + 8 * q + 4 * hi;
+      if (jj < a.dv) *(float4*)(o + jj) = make_float4(acc[tt][4 * q], acc[tt][4 * q + 1], acc[tt][4 * q + 2], acc[tt][4 * q + 3]);
+    }
+  }
+}
+
 extern "C" int ifx_matrix_memory(const void* rows, int dtype, int ld, int q_col, int k_col, int v_col, int g_col, const float* gates, int ldg,
                                  int i_col, int f_col, const float* i_bias, const float* f_bias, float cap, float q_scale,
                                  const float* norm_w, float eps, float* state, long long state_stride, int s_off, const int* q_start,
-                                 const int* q_len, const int* slots, const int* row_req, float* o_raw, float* floor_, float* m_end,
-                                 void* out, int out_dtype, int T, int R, int H, int d, int dv, int ch, int ks, int cols, void* stream) {
+                                 const int* q_len, const int* slots, const int* row_req, float* o_raw, float* nq, float* floor_, float* m_end,
+                                 void* out, int out_dtype, int T, int R, int H, int d, int dv, int ch, int ks, int cols, int n_chunks,
+                                 const int* chunk_req, const int* chunk_t0, const int* chunk_len, const int* req_chunk0, float* token_gates,
+                                 float* chunk_gates, float* chunk_state, void* stream) {
   IFX_REQUIRE(T >= 0 && R >= 0 && H > 0 && d > 0 && dv > 0 && cap > 0.f, "matrix_memory: bad sizes T=%d R=%d H=%d d=%d dv=%d", T, R, H, d, dv);
   IFX_REQUIRE(ks > 0 && ks <= WAVE && (ks & (ks - 1)) == 0 && ch * ks >= d, "matrix_memory: %d threads of %d channels for heads of %d", ks, ch, d);
   IFX_REQUIRE(cols > 0 && cols * ks <= 256, "matrix_memory: %d columns x %d threads do not fit a workgroup of 256", cols, ks);
   IFX_REQUIRE(s_off >= H && s_off % 4 == 0 && state_stride % 4 == 0, "matrix_memory: S must lie at a multiple of 16 bytes behind the maxima");
   IFX_REQUIRE(state_stride >= s_off + (long long)H * (dv + 1) * ch * ks, "matrix_memory: a state row of %lld floats is too short", state_stride);
   IFX_REQUIRE(R <= 65535, "matrix_memory: too many requests for one launch");
-  const size_t lds = (size_t)STAGE * (2 * ch * ks + cols) * sizeof(float);
+  int stage = STAGE;
+  while (stage > 4 && (size_t)stage * (2 * ch * ks + cols) * sizeof(float) > 60 * 1024) stage /= 2;
+  const size_t lds = (size_t)stage * (2 * ch * ks + cols) * sizeof(float);
   IFX_REQUIRE(lds <= 60 * 1024, "matrix_memory: d=%d needs more LDS than a workgroup has", d);
   if (T == 0 || R == 0) return 0;
   MemoryArgs a{rows, ld, q_col, k_col, v_col, g_col, gates, ldg, i_col, f_col, i_bias, f_bias, cap, q_scale, norm_w, eps, state,
-               (size_t)state_stride, s_off, q_start, q_len, slots, row_req, o_raw, floor_, m_end, out, T, R, H, d, dv, ks, cols};
+               (size_t)state_stride, s_off, q_start, q_len, slots, row_req, o_raw, nq, floor_, m_end, out, T, R, H, d, dv, ks, cols, stage};
   const dim3 grid(H * ((dv + cols) / cols), R);        // (dv + 1 columns)
   const int threads = (cols * ks + WAVE - 1) / WAVE * WAVE;
   const unsigned blocks = (unsigned)(((size_t)T * H + 256 / WAVE - 1) / (256 / WAVE));
   hipStream_t s = (hipStream_t)stream;
+  if (n_chunks > 0) {
+    IFX_REQUIRE(dtype == DT_BF16 && d % 8 == 0 && dv % 8 == 0 && ld % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 && v_col % 8 == 0,
+                "matrix_memory: chunks take bfloat16 rows whose heads (d=%d, dv=%d) and columns are multiples of 8", d, dv);
+    IFX_REQUIRE(chunk_req && chunk_t0 && chunk_len && req_chunk0 && token_gates && chunk_gates && chunk_state, "matrix_memory: chunks without their lists");
+    a.m_end = nullptr;           // (the gates' kernel writes the maxima back itself)
+    const size_t HT = (size_t)H * T;
+    const ChunkArgs c{a, chunk_req, chunk_t0, chunk_len, req_chunk0, token_gates, token_gates + HT, token_gates + 2 * HT, chunk_gates,
+                      chunk_gates + (size_t)n_chunks * H, chunk_state, n_chunks, ch * ks};
+    const int jb = (dv + CJ - 1) / CJ, ib = (ch * ks + CI - 1) / CI;
+    const size_t per4 = (size_t)H * (dv + 1) * ch * ks / 4;
+    hipLaunchKernelGGL(memory_gates_kernel, dim3(H, R), dim3(WAVE), 0, s, c);
+    hipLaunchKernelGGL(memory_chunk_sums_kernel, dim3(n_chunks, H, jb * ib), dim3(256), 0, s, c);
+    hipLaunchKernelGGL(memory_combine_kernel, dim3((unsigned)((per4 + 255) / 256), R), dim3(256), 0, s, c);
+    hipLaunchKernelGGL(memory_chunk_out_kernel, dim3(n_chunks, H, jb), dim3(256), 0, s, c);
+    if (out_dtype == DT_BF16) hipLaunchKernelGGL((memory_finish_kernel<bf16_t, bf16_t>), dim3(blocks), dim3(256), 0, s, a);
+    else hipLaunchKernelGGL((memory_finish_kernel<bf16_t, float>), dim3(blocks), dim3(256), 0, s, a);
+    IFX_LAUNCH_CHECK();
+  }
 #define WALK(TY, C) hipLaunchKernelGGL((memory_walk_kernel<TY, C>), grid, dim3(threads), lds, s, a)
 #define BY_CH(TY)                       \
   do {                                  \

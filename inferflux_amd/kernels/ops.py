@@ -1690,6 +1690,13 @@ def _memory_max_floats(n_heads: int) -> int:
     return -(-n_heads // 4) * 4         # the running maxima come first in a state row
 
 
+MEMORY_CHUNK = 64                   # rows of a chunk where long portions are cut into chunks that run side by side
+
+
+def matrix_memory_takes_chunks(dtype: torch.dtype, d: int, dv: int) -> bool:
+    return dtype == torch.bfloat16 and d % 8 == 0 and dv % 8 == 0
+
+
 def matrix_memory_state_floats(n_heads: int, d: int, dv: int) -> int:
     ch, ks, _ = matrix_memory_layout(d, dv)
     return _memory_max_floats(n_heads) + n_heads * (dv + 1) * ch * ks
@@ -1698,12 +1705,16 @@ def matrix_memory_state_floats(n_heads: int, d: int, dv: int) -> int:
 def matrix_memory(rows: torch.Tensor, cols: Tuple[int, int, int, int], gates: torch.Tensor, gate_cols: Tuple[int, int], i_bias: torch.Tensor,
                   f_bias: torch.Tensor, cap: float, norm_weight: torch.Tensor, eps: float, n_heads: int, d: int, dv: int, state: torch.Tensor,
                   q_start: torch.Tensor, q_len: torch.Tensor, slots: torch.Tensor, row_req: torch.Tensor, out_dtype: torch.dtype,
-                  single_tokens: bool = False) -> torch.Tensor:
+                  single_tokens: bool = False, chunks: Optional[Dict[str, object]] = None) -> torch.Tensor:
     """Matrix memory with exponential gates over each request's rows, with the output's norm and gate (see
     csrc/matrix_memory.hip).  ``rows`` [T, ld] holds q, k (n_heads * d each), v and the output gate (n_heads * dv each) at the
     columns ``cols``; ``gates`` float32 [T, ldg] the input and forget gates' numbers (n_heads each) at ``gate_cols``; biases
     float32 [n_heads], ``norm_weight`` float32 [n_heads * dv].  ``state`` float32 [slots, ``matrix_memory_state_floats``], zero
-    for a request that starts.  ``single_tokens``: every request brings one row.  Returns [T, n_heads * dv] in ``out_dtype``."""
+    for a request that starts.  ``single_tokens``: every request brings one row.  Returns [T, n_heads * dv] in ``out_dtype``.
+
+    ``chunks`` (from ``scan_chunks`` with MEMORY_CHUNK rows; bfloat16 rows, see ``matrix_memory_takes_chunks``): the requests'
+    rows in chunks that run side by side on the matrix cores; the same function up to the rounding of float sums taken in
+    another order."""
     _check(rows, "rows", (None, None))
     T, ld = rows.shape
     _check(gates, "gates", (T, None), torch.float32)
@@ -1730,14 +1741,28 @@ def matrix_memory(rows: torch.Tensor, cols: Tuple[int, int, int, int], gates: to
     out = torch.empty((T, HV), dtype=out_dtype, device=rows.device)
     scratch = torch.empty((T * n_heads * (dv + 2) + R * n_heads,), dtype=torch.float32, device=rows.device)
     o_raw = scratch.data_ptr()
-    floor = o_raw + 4 * T * n_heads * (dv + 1)
+    nq = o_raw + 4 * T * n_heads * dv
+    floor = nq + 4 * T * n_heads
     m_end = floor + 4 * T * n_heads
+    n_chunks, lists = 0, (0,) * 7
+    if chunks is not None:
+        if not matrix_memory_takes_chunks(rows.dtype, d, dv) or chunks["rows"] != MEMORY_CHUNK:
+            raise KernelError(f"matrix_memory: chunks of {chunks['rows']} rows of {rows.dtype} with heads of {d} x {dv} (chunks of "
+                              f"{MEMORY_CHUNK} rows of bfloat16, heads of multiples of 8)")
+        n_chunks = chunks["req"].shape[0]
+        for nm in ("req", "t0", "len"):
+            _check(chunks[nm], f"chunks.{nm}", (n_chunks,), torch.int32)
+        _check(chunks["req_chunk0"], "chunks.req_chunk0", (R + 1,), torch.int32)
+        gates_scratch = torch.empty((3 * n_heads * T + 2 * n_heads * n_chunks,), dtype=torch.float32, device=rows.device)
+        chunk_state = torch.empty((n_chunks, n_heads * (dv + 1) * ch * ks), dtype=torch.float32, device=rows.device)
+        lists = (chunks["req"].data_ptr(), chunks["t0"].data_ptr(), chunks["len"].data_ptr(), chunks["req_chunk0"].data_ptr(),
+                 gates_scratch.data_ptr(), gates_scratch.data_ptr() + 12 * n_heads * T, chunk_state.data_ptr())
     _call(load_module("matrix_memory"), "ifx_matrix_memory",
-          (P, I, I, I, I, I, I, P, I, I, I, P, P, F, F, P, F, P, LL, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, P),
+          (P, I, I, I, I, I, I, P, I, I, I, P, P, F, F, P, F, P, LL, I, P, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, P, P, P, P),
           rows.data_ptr(), _dt(rows), ld, q_col, k_col, v_col, g_col, gates.data_ptr(), ldg, i_col, f_col, i_bias.data_ptr(),
           f_bias.data_ptr(), float(cap), float(d) ** -0.5, norm_weight.data_ptr(), float(eps), state.data_ptr(), state.shape[1], s_off,
-          q_start.data_ptr(), q_len.data_ptr(), slots.data_ptr(), row_req.data_ptr(), o_raw, floor, m_end, out.data_ptr(), _DT[out_dtype],
-          T, R, n_heads, d, dv, ch, ks, wg_cols, _stream())
+          q_start.data_ptr(), q_len.data_ptr(), slots.data_ptr(), row_req.data_ptr(), o_raw, nq, floor, m_end, out.data_ptr(), _DT[out_dtype],
+          T, R, n_heads, d, dv, ch, ks, wg_cols, n_chunks, *lists, _stream())
     return out
 
 

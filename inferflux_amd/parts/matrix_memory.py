@@ -30,6 +30,9 @@ from .ffn import concat_weights
 from .plan import ParamSpec, StateSpec
 
 
+CHUNK_MIN_ROWS = 64         # a step that brings some request this many rows or more takes the chunks
+
+
 @register_part("mixer", "matrix_memory")
 class MatrixMemory(Mixer):
     graph_safe = True          # every kernel reads the step's layout from the context's device arrays
@@ -80,7 +83,15 @@ class MatrixMemory(Mixer):
         if state is None:
             raise ValueError(f"{self.name}: the mixer was given no per-request state")
         QK, V, nh, dtype = self.qk_width, self.v_width, self.n_heads, h.dtype
-        if ops.streams_weight(h.shape[0], self.w_in):
+        # A prompt's portion walked token by token leaves most of the chip idle: in bfloat16 long portions are cut into chunks
+        # that run side by side.  In 32-bit the walk stays in one piece, so that a token's sums do not depend on where its
+        # request was cut.  (Steps of single tokens never take the chunks: a captured layout keeps its launches.)
+        chunks = None
+        if (ctx.n_tokens > ctx.n_requests and ops.matrix_memory_takes_chunks(dtype, self.head_dim, self.v_head_dim)
+                and int(ctx.h_q_len.max()) >= CHUNK_MIN_ROWS):
+            chunks = ctx.derived(("scan_chunks", ops.MEMORY_CHUNK),
+                                 lambda: ops.scan_chunks(ctx.h_q_start, ctx.h_q_len, ops.MEMORY_CHUNK, ctx.device))
+        if chunks is None and ops.streams_weight(h.shape[0], self.w_in):
             # few rows: one product whose float sums are read as they are
             rows = ops.linear(h, self.w_in, out_dtype=torch.float32)
             gates, i_col = rows, 2 * QK + 2 * V
@@ -91,7 +102,7 @@ class MatrixMemory(Mixer):
             t.mark("mixer.project")
         y = ops.matrix_memory(rows, (0, QK, 2 * QK, 2 * QK + V), gates, (i_col, i_col + nh), self.i_bias, self.f_bias, self.gate_cap,
                               self.norm_w, self.norm_eps, nh, self.head_dim, self.v_head_dim, state, ctx.q_start, ctx.q_len,
-                              ctx.state_slots, ctx.row_req, dtype, single_tokens=ctx.n_tokens == ctx.n_requests)
+                              ctx.state_slots, ctx.row_req, dtype, single_tokens=ctx.n_tokens == ctx.n_requests, chunks=chunks)
         if t is not None:
             t.mark("mixer.scan")
         if sink is not None and ops.adds_into_stream(y.shape[0], self.w_o, sink.norm_weight):

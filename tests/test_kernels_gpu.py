@@ -1480,8 +1480,23 @@ def test_scaled_rows_are_refused_where_no_kernel_applies_them():
         ops.linear(scaled, torch.randn(8, 64, device=DEV).bfloat16())               # a bare tensor
     with pytest.raises(ops.KernelError, match="linear_into_stream"):
         ops.linear_into_stream(torch.zeros(17, 32, dtype=BF16, device=DEV), lw, torch.zeros(17, 64, device=DEV), nw.to(DEV), 1e-5)
-    with pytest.raises(ops.KernelError, match="linear_into_stream"):               # a float32 norm weight
-        ops.linear_into_stream(x.to(DEV), lw, stream.to(DEV), nw.float().to(DEV), 1e-5)
+
+
+@pytest.mark.parametrize("M,N,K", [(1, 64, 32), (7, 256, 512), (16, 1000, 200)])
+def test_a_float_norm_weight_prepares_the_same_rows(M, N, K):
+    """A norm's weight formed at load (one plus what the file holds) stays float: with the values of a bfloat16 weight it gives
+    that weight's bits, and a difference that bfloat16 has no room for is not lost."""
+    x, w, stream, nw, lw = _stream_case(M, N, K, 34, True)
+    a, b = stream.to(DEV).clone(), stream.to(DEV).clone()
+    one = ops.linear_into_stream(x.to(DEV), lw, a, nw.to(DEV), 1e-5)
+    two = ops.linear_into_stream(x.to(DEV), lw, b, nw.float().to(DEV), 1e-5)
+    assert torch.equal(a, b) and torch.equal(one.rows, two.rows) and torch.equal(one.pieces, two.pieces)
+    fine = (1.0 + 0.001 * torch.randn(N, generator=gen(5))).to(DEV)
+    three = ops.linear_into_stream(x.to(DEV), lw, stream.to(DEV).clone(), fine, 1e-5)
+    assert torch.equal(three.rows, (a * fine).to(BF16))
+    table, ids = torch.randn(20, N, generator=gen(6)).to(BF16).to(DEV), torch.arange(M, dtype=torch.int32, device=DEV)
+    out, rows = ops.embedding_scaled(ids, table, fine, 1e-5)
+    assert torch.equal(rows.rows, (out * fine).to(BF16))
 
 
 @pytest.mark.parametrize("M", [1, 7, 16, 33, 64])
