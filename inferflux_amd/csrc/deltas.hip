@@ -8,15 +8,15 @@
 IFX_DEFINE_LAST_ERROR()
 
 #define MAX_TERMS 6
+#define MAX_PIECES 64        // tensors, vectors and single slices of all terms
 
-struct Term { const void* p; size_t slice_stride; int dtype, n_slices, row_stride; float scale; };
-struct Terms { Term t[MAX_TERMS]; int n; };
+// What is added, piece by piece: a slice of a term is a piece of its own, so that the loads of many are on their way at once.
+struct Piece { const void* p; int dtype, row_stride; float scale; };
+struct Pieces { Piece t[MAX_PIECES]; int n; };
 
-__device__ __forceinline__ float term_at(const Term& k, size_t row, int i) {
-  const size_t at = row * k.row_stride + i;
-  float v = load_dyn(k.p, k.dtype, at);
-  for (int s = 1; s < k.n_slices; ++s) v += ((const float*)k.p)[(size_t)s * k.slice_stride + at];
-  return v * k.scale;
+__device__ __forceinline__ float pieces_at(const Pieces& pieces, size_t row, int i, float x) {
+  for (int k = 0; k < pieces.n; ++k) x = fmaf(load_dyn(pieces.t[k].p, pieces.t[k].dtype, row * pieces.t[k].row_stride + i), pieces.t[k].scale, x);
+  return x;
 }
 typedef __attribute__((__vector_size__(4 * sizeof(__bf16)))) __bf16 dl_bf16x4;
 __device__ __forceinline__ void dl_load4(const void* p, int dtype, size_t at, float* v) {
@@ -36,33 +36,35 @@ __device__ __forceinline__ void dl_store4(bf16_t* p, const float* v) {
   for (int e = 0; e < 4; ++e) t[e] = (__bf16)v[e];
   *(dl_bf16x4*)p = t;
 }
-// x[v][..] += the terms at columns 4 (threadIdx.x + 256 v) of ``row``
+// x[v][..] += the pieces at columns 4 (threadIdx.x + 256 v) of ``row``, AT_ONCE of them asked for before the first is added
 template <int NV>
-__device__ __forceinline__ void add_terms4(const Terms& terms, size_t row, int H, float x[NV][4]) {
-  for (int k = 0; k < terms.n; ++k) {
-    const Term& term = terms.t[k];
-    float d[NV][4];
-    for (int s = 0; s < term.n_slices; ++s) {
+__device__ __forceinline__ void add_pieces4(const Pieces& pieces, size_t row, int H, float x[NV][4]) {
+  constexpr int AT_ONCE = NV <= 2 ? 8 : (NV <= 4 ? 4 : 2);
+  for (int k0 = 0; k0 < pieces.n; k0 += AT_ONCE) {
+    float d[AT_ONCE][NV][4];
+#pragma unroll
+    for (int u = 0; u < AT_ONCE; ++u) {
+      const Piece& k = pieces.t[min(k0 + u, pieces.n - 1)];
 #pragma unroll
       for (int v = 0; v < NV; ++v) {
         const int i = 4 * (threadIdx.x + 256 * v);
-        if (i >= H) continue;
-        float p[4];
-        dl_load4(term.p, term.dtype, (size_t)s * term.slice_stride + row * term.row_stride + i, p);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) d[v][e] = s == 0 ? p[e] : d[v][e] + p[e];
+        if (i < H && k0 + u < pieces.n) dl_load4(k.p, k.dtype, row * k.row_stride + i, d[u][v]);
+        else d[u][v][0] = d[u][v][1] = d[u][v][2] = d[u][v][3] = 0.f;
       }
     }
 #pragma unroll
-    for (int v = 0; v < NV; ++v)
-      if (4 * (threadIdx.x + 256 * v) < H)
+    for (int u = 0; u < AT_ONCE; ++u) {
+      const float scale = pieces.t[min(k0 + u, pieces.n - 1)].scale;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) x[v][e] = fmaf(d[v][e], term.scale, x[v][e]);
+      for (int v = 0; v < NV; ++v)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[v][e] = fmaf(d[u][v][e], scale, x[v][e]);
+    }
   }
 }
 
 template <typename TO, int NV>
-__global__ __launch_bounds__(256) void add_terms_rmsnorm4_kernel(float* __restrict__ stream, Terms terms, const void* __restrict__ weight,
+__global__ __launch_bounds__(256) void add_terms_rmsnorm4_kernel(float* __restrict__ stream, Pieces pieces, const void* __restrict__ weight,
                                                                  int weight_dtype, TO* __restrict__ out, const int* __restrict__ rows, int H,
                                                                  float eps, int write_back) {
   __shared__ float red[16];
@@ -74,7 +76,7 @@ __global__ __launch_bounds__(256) void add_terms_rmsnorm4_kernel(float* __restri
     if (i < H) dl_load4(stream, DT_F32, src * H + i, x[v]);
     else x[v][0] = x[v][1] = x[v][2] = x[v][3] = 0.f;
   }
-  add_terms4<NV>(terms, src, H, x);
+  add_pieces4<NV>(pieces, src, H, x);
   float ss = 0.f;
 #pragma unroll
   for (int v = 0; v < NV; ++v) {
@@ -98,17 +100,13 @@ __global__ __launch_bounds__(256) void add_terms_rmsnorm4_kernel(float* __restri
 
 // any width: the sum is formed twice where it is not written back
 template <typename TO>
-__global__ __launch_bounds__(256) void add_terms_rmsnorm_kernel(float* __restrict__ stream, Terms terms, const void* __restrict__ weight,
+__global__ __launch_bounds__(256) void add_terms_rmsnorm_kernel(float* __restrict__ stream, Pieces pieces, const void* __restrict__ weight,
                                                                 int weight_dtype, TO* __restrict__ out, const int* __restrict__ rows, int H,
                                                                 float eps, int write_back) {
   __shared__ float red[16];
   const size_t src = rows ? (size_t)rows[blockIdx.x] : (size_t)blockIdx.x;
   float* res = stream + src * H;
-  auto at = [&](int i) {
-    float x = res[i];
-    for (int k = 0; k < terms.n; ++k) x += term_at(terms.t[k], src, i);
-    return x;
-  };
+  auto at = [&](int i) { return pieces_at(pieces, src, i, res[i]); };
   float ss = 0.f;
   for (int i = threadIdx.x; i < H; i += 256) {
     const float x = at(i);
@@ -123,15 +121,14 @@ __global__ __launch_bounds__(256) void add_terms_rmsnorm_kernel(float* __restric
 }
 
 template <typename TO>
-__global__ __launch_bounds__(256) void join_stream_kernel(const float* __restrict__ stream, Terms terms, const float* __restrict__ other,
+__global__ __launch_bounds__(256) void join_stream_kernel(const float* __restrict__ stream, Pieces pieces, const float* __restrict__ other,
                                                           TO* __restrict__ out, int H) {
   const size_t t = blockIdx.x;
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c >= 2 * H) return;
   float x;
   if (c < H) {
-    x = stream[t * H + c];
-    for (int k = 0; k < terms.n; ++k) x += term_at(terms.t[k], t, c);
+    x = pieces_at(pieces, t, c, stream[t * H + c]);
   } else {
     x = other[t * H + c - H];
   }
@@ -139,13 +136,15 @@ __global__ __launch_bounds__(256) void join_stream_kernel(const float* __restric
 }
 
 // The terms as arrays on the host: pointers, element types, slices, elements between slices and rows, factors.
-static int gather_terms(Terms& out, int n, const void* const* p, const int* dtype, const int* n_slices, const long long* slice_stride,
+static int gather_terms(Pieces& out, int n, const void* const* p, const int* dtype, const int* n_slices, const long long* slice_stride,
                         const int* row_stride, const float* scale) {
+  out.n = 0;
   if (n < 0 || n > MAX_TERMS) return 0;
-  out.n = n;
   for (int k = 0; k < n; ++k) {
     if (!p[k] || n_slices[k] < 1 || (n_slices[k] > 1 && dtype[k] != DT_F32) || (dtype[k] != DT_F32 && dtype[k] != DT_BF16)) return 0;
-    out.t[k] = Term{p[k], (size_t)slice_stride[k], dtype[k], n_slices[k], row_stride[k], scale[k]};
+    if (out.n + n_slices[k] > MAX_PIECES) return 0;
+    for (int s = 0; s < n_slices[k]; ++s)
+      out.t[out.n++] = Piece{(const char*)p[k] + (size_t)s * slice_stride[k] * sizeof(float), dtype[k], row_stride[k], scale[k]};
   }
   return 1;
 }
@@ -157,18 +156,18 @@ extern "C" int ifx_add_terms_rmsnorm(float* stream_io, int n_terms, const void* 
   IFX_REQUIRE(n_rows >= 0 && H > 0, "add_terms_rmsnorm: bad sizes rows=%d H=%d", n_rows, H);
   IFX_REQUIRE(!(rows && write_back), "add_terms_rmsnorm: a row gather cannot write the stream back");
   IFX_REQUIRE(out_dtype == DT_F32 || out_dtype == DT_BF16, "add_terms_rmsnorm: unknown out dtype %d", out_dtype);
-  Terms terms;
-  IFX_REQUIRE(gather_terms(terms, n_terms, p, dtype, n_slices, slice_stride, row_stride, scale), "add_terms_rmsnorm: bad terms (%d, at most %d)", n_terms, MAX_TERMS);
+  Pieces pieces;
+  IFX_REQUIRE(gather_terms(pieces, n_terms, p, dtype, n_slices, slice_stride, row_stride, scale), "add_terms_rmsnorm: bad terms (%d, at most %d, of %d slices together)", n_terms, MAX_TERMS, MAX_PIECES);
   if (n_rows == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-#define GO4(TO, NV) hipLaunchKernelGGL((add_terms_rmsnorm4_kernel<TO, NV>), dim3(n_rows), dim3(256), 0, s, stream_io, terms, weight, weight_dtype, (TO*)out, rows, H, eps, write_back)
+#define GO4(TO, NV) hipLaunchKernelGGL((add_terms_rmsnorm4_kernel<TO, NV>), dim3(n_rows), dim3(256), 0, s, stream_io, pieces, weight, weight_dtype, (TO*)out, rows, H, eps, write_back)
 #define GO(TO)                                          \
   do {                                                  \
     if (H % 4 == 0 && H <= 1024) GO4(TO, 1);            \
     else if (H % 4 == 0 && H <= 2048) GO4(TO, 2);       \
     else if (H % 4 == 0 && H <= 4096) GO4(TO, 4);       \
     else if (H % 4 == 0 && H <= 8192) GO4(TO, 8);       \
-    else hipLaunchKernelGGL(add_terms_rmsnorm_kernel<TO>, dim3(n_rows), dim3(256), 0, s, stream_io, terms, weight, weight_dtype, (TO*)out, rows, H, eps, write_back); \
+    else hipLaunchKernelGGL(add_terms_rmsnorm_kernel<TO>, dim3(n_rows), dim3(256), 0, s, stream_io, pieces, weight, weight_dtype, (TO*)out, rows, H, eps, write_back); \
   } while (0)
   if (out_dtype == DT_F32) GO(float);
   else GO(bf16_t);
@@ -181,13 +180,13 @@ extern "C" int ifx_join_stream(const float* x, int n_terms, const void* const* p
                                const long long* slice_stride, const int* row_stride, const float* scale, const float* other, void* out,
                                int out_dtype, int T, int H, void* stream) {
   IFX_REQUIRE(T >= 0 && H > 0, "join_stream: bad sizes T=%d H=%d", T, H);
-  Terms terms;
-  IFX_REQUIRE(gather_terms(terms, n_terms, p, dtype, n_slices, slice_stride, row_stride, scale), "join_stream: bad terms (%d, at most %d)", n_terms, MAX_TERMS);
+  Pieces pieces;
+  IFX_REQUIRE(gather_terms(pieces, n_terms, p, dtype, n_slices, slice_stride, row_stride, scale), "join_stream: bad terms (%d, at most %d, of %d slices together)", n_terms, MAX_TERMS, MAX_PIECES);
   if (T == 0) return 0;
   const dim3 grid(T, (2 * H + 255) / 256);
   hipStream_t s = (hipStream_t)stream;
-  if (out_dtype == DT_F32) hipLaunchKernelGGL(join_stream_kernel<float>, grid, dim3(256), 0, s, x, terms, other, (float*)out, H);
-  else if (out_dtype == DT_BF16) hipLaunchKernelGGL(join_stream_kernel<bf16_t>, grid, dim3(256), 0, s, x, terms, other, (bf16_t*)out, H);
+  if (out_dtype == DT_F32) hipLaunchKernelGGL(join_stream_kernel<float>, grid, dim3(256), 0, s, x, pieces, other, (float*)out, H);
+  else if (out_dtype == DT_BF16) hipLaunchKernelGGL(join_stream_kernel<bf16_t>, grid, dim3(256), 0, s, x, pieces, other, (bf16_t*)out, H);
   else IFX_FAIL("join_stream: unknown out dtype %d", out_dtype);
   IFX_LAUNCH_CHECK();
 }

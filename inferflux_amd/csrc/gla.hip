@@ -259,7 +259,8 @@ static int launch_gla(const GlaArgs& a, int R, int n_chunks, const int* req_chun
   // load, so a head of few values still gets a thread per key channel.
   constexpr int MAX_COLS = DP <= 16 ? 4 : (DP <= 32 ? 2 : 1);
   const auto threads_for = [&](int cols) { return ((max((a.dv + cols - 1) / cols * a.parts, a.d) + WAVE - 1) / WAVE) * WAVE; };
-  int cols_chunk = min(2, MAX_COLS);
+  // (time mixing's heads have as few values as keys: with two columns a thread a head of 64 x 64 would be two waves)
+  int cols_chunk = TIME_MIX && threads_for(1) <= 256 ? 1 : min(2, MAX_COLS);
   while (cols_chunk < MAX_COLS && threads_for(cols_chunk) > GLA_MAX_THREADS(DP)) cols_chunk *= 2;
   const int cols_walk = cols_chunk;
   IFX_REQUIRE(threads_for(cols_chunk) <= GLA_MAX_THREADS(DP), "gla_scan: %d threads a head with %d channels each (at most %d)",

@@ -25,9 +25,9 @@
 // from a chunk's start and m0 the maximum before the chunk, for tokens s <= t of a chunk
 //   o_t = exp(F_t + m0 - m_t) S0^T q_t + sum_s exp(F_t - F_s + i_s - m_t) (q_t . k_s) v_s          (every exponent is <= 0)
 //   S_end = exp(F_L + m0 - m_L) S0 + sum_s exp(F_L - F_s + i_s - m_L) k_s v_s^T
-// in four launches: the gates and maxima of all tokens (a wave per request and head, exact for the whole portion, so nothing is
-// ever rescaled), each chunk's own sum of outer products, the walk over a request's chunks that leaves S0 of every chunk, and
-// the read-outs.  q, k and v are the projections' bfloat16 numbers as they are; what is float on the way into a product (S0,
+// in four launches: the gates and maxima of all tokens (exact for the whole portion, so nothing is ever rescaled), each chunk's
+// own sum of outer products, the walk over a request's chunks that leaves S0 of every chunk, and the read-outs, which finish
+// heads of up to CJ values themselves (the second kernel above does it for wider ones).  q, k and v are the projections' bfloat16 numbers as they are; what is float on the way into a product (S0,
 // the weighted keys, the weighted scores) goes in as two bfloat16 numbers, the rounded one and the rest, so that nothing of
 // the recurrence is rounded to 16 bits.  The normaliser's sums are plain float.
 #include "common.h"
@@ -202,50 +202,53 @@ __device__ __forceinline__ bf16x8 zero8() {
   return z;
 }
 
-// A wave per (request, head): a chunk's tokens a lane each.
-__global__ __launch_bounds__(WAVE) void memory_gates_kernel(ChunkArgs c) {
+// A workgroup per (request, head), a chunk a wave and a token a lane: the waves scan their chunks side by side, the chunks' sums
+// meet in LDS, and every wave walks those before its own for the maximum its chunk starts from.
+#define GATE_WAVES 16
+__global__ __launch_bounds__(GATE_WAVES * WAVE) void memory_gates_kernel(ChunkArgs c) {
   const MemoryArgs& a = c.a;
-  const int h = blockIdx.x, r = blockIdx.y, lane = threadIdx.x;
+  __shared__ float sum_f[2][GATE_WAVES], best[2][GATE_WAVES];      // two sets in turns: one barrier a round is enough
+  const int h = blockIdx.x, r = blockIdx.y, lane = threadIdx.x % WAVE, wid = threadIdx.x / WAVE, nw = blockDim.x / WAVE;
   const int n = a.q_len[r];
   if (n <= 0) return;
   const int t0 = a.q_start[r], c0 = c.req_chunk0[r];
   float* m_state = a.state + (size_t)a.slots[r] * a.state_stride + h;
-  float m = *m_state;
+  float m = *m_state;                  // the maximum before the round's first chunk, the same in every wave
   const float ib = a.i_bias[h], fb = a.f_bias[h];
-  float gi = 0.f, gf = 0.f;
-  auto fetch = [&](int base) {
-    if (base + lane < n) {
-      const float* g = a.gates + (size_t)(t0 + base + lane) * a.ldg;
-      gi = g[a.i_col + h]; gf = g[a.f_col + h];
-    }
-  };
-  fetch(0);
-  for (int base = 0, k = 0; base < n; base += CL, ++k) {
-    const int cnt = min(CL, n - base);
+  for (int base = 0, round = 0; base < n; base += nw * CL, ++round) {
+    const int at0 = base + wid * CL, cnt = min(CL, n - at0);        // (a wave behind the last chunk has none: cnt <= 0)
     const bool in = lane < cnt;
-    const float li = in ? soft_cap(gi + ib, a.cap) : -INFINITY;
-    const float lf = in ? log_sigmoid(soft_cap(gf + fb, a.cap)) : 0.f;
-    fetch(base + CL);                  // the next chunk's are on their way during the scan
+    const float* g = a.gates + (size_t)(t0 + (in ? at0 + lane : 0)) * a.ldg;
+    const float li = in ? soft_cap(g[a.i_col + h] + ib, a.cap) : -INFINITY;
+    const float lf = in ? log_sigmoid(soft_cap(g[a.f_col + h] + fb, a.cap)) : 0.f;
     float F = lf, M = li;
 #pragma unroll
     for (int o = 1; o < CL; o <<= 1) {
       const float Fp = __shfl_up(F, o, WAVE), Mp = __shfl_up(M, o, WAVE);
       if (lane >= o) { M = fmaxf(Mp + F, M); F += Fp; }
     }
-    const float mt = fmaxf(m + F, M);
+    float (&sf)[GATE_WAVES] = sum_f[round & 1], (&sb)[GATE_WAVES] = best[round & 1];
+    if (lane == WAVE - 1) { sf[wid] = F; sb[wid] = M; }              // (lanes behind the chunk's end add nothing)
+    __syncthreads();
+    float m_here = m;
+    for (int w = 0; w < nw; ++w) {
+      if (w == wid) m_here = m;
+      m = fmaxf(m + sf[w], sb[w]);                                   // (a wave without tokens: m + 0 against -inf)
+    }
+    if (cnt <= 0) continue;
+    const float mt = fmaxf(m_here + F, M);
     if (in) {
-      const size_t at = (size_t)h * a.T + t0 + base + lane;
+      const size_t at = (size_t)h * a.T + t0 + at0 + lane;
       c.cum_f[at] = F; c.log_i[at] = li; c.m[at] = mt;
-      a.floor[(size_t)(t0 + base + lane) * a.H + h] = expf(-mt);
+      a.floor[(size_t)(t0 + at0 + lane) * a.H + h] = expf(-mt);
     }
-    const float m_last = __shfl(mt, cnt - 1, WAVE), F_last = __shfl(F, cnt - 1, WAVE);
-    if (lane == 0) {
-      c.m0[(size_t)(c0 + k) * a.H + h] = m;
-      c.keep[(size_t)(c0 + k) * a.H + h] = expf(F_last + m - m_last);
+    if (lane == cnt - 1) {
+      const size_t at = (size_t)(c0 + round * nw + wid) * a.H + h;
+      c.m0[at] = m_here;
+      c.keep[at] = expf(F + m_here - mt);
     }
-    m = m_last;
   }
-  if (lane == 0) *m_state = m;
+  if (threadIdx.x == 0) *m_state = m;
 }
 
 // value columns j0 .. of head h's v, tokens in pairs, as rows [column][token] of LDS (zeros beyond dv and beyond the chunk)
@@ -360,13 +363,20 @@ __global__ __launch_bounds__(256) void memory_combine_kernel(ChunkArgs c) {
   *slot = S;
 }
 
-// The read-outs of a chunk's tokens for CJ columns of a head.
+// The read-outs of a chunk's tokens for CJ columns of a head.  FINISH (dv <= CJ): the head's norm, weight and gate as well, from
+// the read-outs in LDS; else they go to o_raw and nq.
+#define OTP (CJ + 4)         // a token's read-outs in LDS
+template <typename TO, bool FINISH>
 __global__ __launch_bounds__(256) void memory_chunk_out_kernel(ChunkArgs c) {
   const MemoryArgs& a = c.a;
-  __shared__ __attribute__((aligned(16))) bf16_t vt[CJ][CLP];
-  __shared__ __attribute__((aligned(16))) bf16_t ph[CL][CLP];
-  __shared__ __attribute__((aligned(16))) bf16_t pl[CL][CLP];
-  __shared__ float Fs[CL], is[CL], ms[CL], row_sum[2][CL];
+  __shared__ __attribute__((aligned(16))) union {
+    struct { bf16_t vt[CJ][CLP], ph[CL][CLP], pl[CL][CLP]; } w;
+    float ot[CL][OTP];
+  } pool;
+  bf16_t (&vt)[CJ][CLP] = pool.w.vt;
+  bf16_t (&ph)[CL][CLP] = pool.w.ph;
+  bf16_t (&pl)[CL][CLP] = pool.w.pl;
+  __shared__ float Fs[CL], is[CL], ms[CL], row_sum[2][CL], inv_den[CL];
   const int chunk = blockIdx.x, h = blockIdx.y, j0 = blockIdx.z * CJ;
   const int t0 = c.chunk_t0[chunk], len = c.chunk_len[chunk], tid = threadIdx.x, d = a.d;
   const int wave = tid / WAVE, lane = tid % WAVE, l32 = lane & 31, hi = lane >> 5;
@@ -421,11 +431,13 @@ __global__ __launch_bounds__(256) void memory_chunk_out_kernel(ChunkArgs c) {
       for (int i = part; i < d; i += 4) nq = fmaf((float)qb[(size_t)t * a.ld + i], S0[(size_t)a.dv * c.dpad + i], nq);
     nq += __shfl_xor(nq, 1, WAVE);
     nq += __shfl_xor(nq, 2, WAVE);
-    if (part == 0 && t < len)
-      a.nq[(size_t)(t0 + t) * a.H + h] = nq * a.q_scale * expf(Fs[t] + m0 - ms[t]) + row_sum[0][t] + row_sum[1][t];
+    nq = nq * a.q_scale * expf(Fs[t] + m0 - ms[t]) + row_sum[0][t] + row_sum[1][t];
+    if (FINISH) { if (part == 0) inv_den[t] = 1.0f / (fmaxf(fabsf(nq), expf(-ms[t])) + 1e-6f); }
+    else if (part == 0 && t < len) a.nq[(size_t)(t0 + t) * a.H + h] = nq;
   }
   const int j = j0 + 32 * wave + l32;
-  if (j0 + 32 * wave >= a.dv) return;
+  const bool mine = j0 + 32 * wave < a.dv;         // (the same for the whole wave)
+  if (!FINISH && !mine) return;
   floatx16 acc[2];
 #pragma unroll
   for (int tt = 0; tt < 2; ++tt)
@@ -433,7 +445,8 @@ __global__ __launch_bounds__(256) void memory_chunk_out_kernel(ChunkArgs c) {
     for (int e = 0; e < 16; ++e) acc[tt][e] = 0.f;
   // what the chunk starts from: S0's rows are asked for as floats and go in as two bfloat16 numbers
   const float* Srow = S0 + (size_t)min(j, a.dv - 1) * c.dpad;
-  for (int k = 8 * hi; k < d + 8 * hi; k += 16) {
+  const int d_here = mine ? d : 0;
+  for (int k = 8 * hi; k < d_here + 8 * hi; k += 16) {
     bf16x8 sh = zero8(), sl = zero8();
     if (k < d) {
       const float4 x = *(const float4*)(Srow + k), y = *(const float4*)(Srow + k + 4);
@@ -467,6 +480,48 @@ __global__ __launch_bounds__(256) void memory_chunk_out_kernel(ChunkArgs c) {
     }
   }
   // acc[tt][e]: column j0 + 32 wave + 8 (e / 4) + 4 hi + e % 4 of token 32 tt + l32 (dv is a multiple of 8: runs of four are whole)
+  if (FINISH) {
+    __syncthreads();             // everyone is done with the columns and the weighted scores: the read-outs take their place
+    if (mine)
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt)
+#pragma unroll
+        for (int q = 0; q < 4; ++q)
+          *(float4*)&pool.ot[32 * tt + l32][32 * wave + 8 * q + 4 * hi] =
+              make_float4(acc[tt][4 * q], acc[tt][4 * q + 1], acc[tt][4 * q + 2], acc[tt][4 * q + 3]);
+    __syncthreads();
+    // four threads a token, each every fourth run of eight columns
+    const int t = tid >> 2, part = tid & 3;
+    const float* o = pool.ot[t];
+    const float id = inv_den[t];
+    float ss = 0.f;
+    for (int g = 8 * part; g < a.dv; g += 32)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) { const float v = o[g + e] * id; ss = fmaf(v, v, ss); }
+    ss += __shfl_xor(ss, 1, WAVE);
+    ss += __shfl_xor(ss, 2, WAVE);
+    if (t >= len) return;
+    const float f = id / sqrtf(ss / (float)a.dv + a.eps);
+    const size_t row = (size_t)(t0 + t);
+    for (int g = 8 * part; g < a.dv; g += 32) {
+      const bf16x8 gate = *(const bf16x8*)(rows + row * a.ld + a.g_col + (size_t)h * a.dv + g);
+      const float* w = a.norm_w + (size_t)h * a.dv + g;
+      TO* out = (TO*)a.out + (row * a.H + h) * a.dv + g;
+      float y[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) y[e] = o[g + e] * f * w[e] / (1.0f + expf(-(float)gate[e]));
+      if (sizeof(TO) == 2) {
+        bf16x8 z;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) z[e] = (__bf16)y[e];
+        *(bf16x8*)out = z;
+      } else {
+        *(float4*)out = make_float4(y[0], y[1], y[2], y[3]);
+        *(float4*)((float*)out + 4) = make_float4(y[4], y[5], y[6], y[7]);
+      }
+    }
+    return;
+  }
 #pragma unroll
   for (int tt = 0; tt < 2; ++tt) {
     const int t = 32 * tt + l32;
@@ -514,10 +569,16 @@ extern "C" int ifx_matrix_memory(const void* rows, int dtype, int ld, int q_col,
                       chunk_gates + (size_t)n_chunks * H, chunk_state, n_chunks, ch * ks};
     const int jb = (dv + CJ - 1) / CJ, ib = (ch * ks + CI - 1) / CI;
     const size_t per4 = (size_t)H * (dv + 1) * ch * ks / 4;
-    hipLaunchKernelGGL(memory_gates_kernel, dim3(H, R), dim3(WAVE), 0, s, c);
+    const int gate_waves = min(GATE_WAVES, max(1, n_chunks - R + 1));        // (no request has more chunks than this)
+    hipLaunchKernelGGL(memory_gates_kernel, dim3(H, R), dim3(gate_waves * WAVE), 0, s, c);
     hipLaunchKernelGGL(memory_chunk_sums_kernel, dim3(n_chunks, H, jb * ib), dim3(256), 0, s, c);
     hipLaunchKernelGGL(memory_combine_kernel, dim3((unsigned)((per4 + 255) / 256), R), dim3(256), 0, s, c);
-    hipLaunchKernelGGL(memory_chunk_out_kernel, dim3(n_chunks, H, jb), dim3(256), 0, s, c);
+    if (dv <= CJ && g_col % 8 == 0) {
+      if (out_dtype == DT_BF16) hipLaunchKernelGGL((memory_chunk_out_kernel<bf16_t, true>), dim3(n_chunks, H, 1), dim3(256), 0, s, c);
+      else hipLaunchKernelGGL((memory_chunk_out_kernel<float, true>), dim3(n_chunks, H, 1), dim3(256), 0, s, c);
+      IFX_LAUNCH_CHECK();
+    }
+    hipLaunchKernelGGL((memory_chunk_out_kernel<float, false>), dim3(n_chunks, H, jb), dim3(256), 0, s, c);
     if (out_dtype == DT_BF16) hipLaunchKernelGGL((memory_finish_kernel<bf16_t, bf16_t>), dim3(blocks), dim3(256), 0, s, a);
     else hipLaunchKernelGGL((memory_finish_kernel<bf16_t, float>), dim3(blocks), dim3(256), 0, s, a);
     IFX_LAUNCH_CHECK();

@@ -2,7 +2,7 @@
 //   shifted_mixes   out[s][t][c] = h[t][c] + (h'[t][c] - h[t][c]) mu[s][c] for S sources s, h' the request's row before t: the row
 //                   before in this step, or the last row of the request's last step, kept in its state (zeros for a request
 //                   that starts), which is replaced by this step's last row
-//   lowrank_tanh    z[t][c] = sum_r W[c][r] tanh(a[t][r]), float sums
+//   lowrank_tanh    z[t][c] = sum_r W[r][c] tanh(a[t][r]), float sums
 // All arithmetic is float.
 #include "common.h"
 
@@ -86,53 +86,86 @@ extern "C" int ifx_shifted_mixes(const void* h, int dtype, const float* mu, floa
   IFX_LAUNCH_CHECK();
 }
 
-// A workgroup takes ROWS rows and 256 output channels: tanh of the rows' numbers in LDS, a channel a thread, whose weights are
-// read once for all the rows.
-#define LR_ROWS 8
-template <typename T>
-__global__ __launch_bounds__(256) void lowrank_tanh_kernel(const float* __restrict__ a, int lda, const T* __restrict__ w, float* __restrict__ z,
-                                                           int rows, int rank, int C) {
-  extern __shared__ float th[];              // [LR_ROWS][rank]
-  const int t0 = blockIdx.x * LR_ROWS, n = min(LR_ROWS, rows - t0);
-  for (int x = threadIdx.x; x < LR_ROWS * rank; x += 256) {
+// ``w`` is W transposed, [rank][C], so that neighbouring lanes read neighbouring channels.  A workgroup takes ROWS rows and 128
+// output channels, two a lane; tanh of the rows' numbers lies in LDS.  Its four waves share the rank, a quarter each, and their
+// sums meet in LDS in wave order.
+template <typename T> __device__ __forceinline__ void tm_load2(const T* p, float& a, float& b);
+template <> __device__ __forceinline__ void tm_load2<float>(const float* p, float& a, float& b) { const float2 t = *(const float2*)p; a = t.x; b = t.y; }
+template <> __device__ __forceinline__ void tm_load2<bf16_t>(const bf16_t* p, float& a, float& b) {
+  typedef __attribute__((__vector_size__(2 * sizeof(__bf16)))) __bf16 bf16x2;
+  const bf16x2 t = *(const bf16x2*)p;
+  a = (float)t[0]; b = (float)t[1];
+}
+
+#define LR_WAVES 4
+template <typename T, int ROWS>
+__global__ __launch_bounds__(LR_WAVES * WAVE) void lowrank_tanh_kernel(const float* __restrict__ a, int lda, const T* __restrict__ w,
+                                                                      float* __restrict__ z, int rows, int rank, int C) {
+  extern __shared__ __attribute__((aligned(16))) float lr_lds[];       // tanh [rank][ROWS], then the waves' sums [LR_WAVES - 1][ROWS][128]
+  float* th = lr_lds;
+  float* part = lr_lds + rank * ROWS;
+  const int t0 = blockIdx.x * ROWS, n = min(ROWS, rows - t0), wid = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  for (int x = threadIdx.x; x < ROWS * rank; x += LR_WAVES * WAVE) {
     const int tt = x / rank, r = x - tt * rank;
-    th[x] = tt < n ? tanhf(a[(size_t)(t0 + tt) * lda + r]) : 0.f;
+    th[r * ROWS + tt] = tt < n ? tanhf(a[(size_t)(t0 + tt) * lda + r]) : 0.f;
   }
   __syncthreads();
-  const int c = blockIdx.y * 256 + threadIdx.x;
-  if (c >= C) return;
-  float acc[LR_ROWS];
+  const int c = blockIdx.y * 128 + 2 * lane;          // (C is even where two channels are read at once)
+  const bool both = c + 1 < C && C % 2 == 0;
+  float acc[ROWS][2];
 #pragma unroll
-  for (int i = 0; i < LR_ROWS; ++i) acc[i] = 0.f;
-  const T* wc = w + (size_t)c * rank;
-  if (rank % 4 == 0) {
-    for (int r = 0; r < rank; r += 4) {
-      float wv[4];
-      tm_load4<T>(wc + r, wv);
-#pragma unroll
-      for (int i = 0; i < LR_ROWS; ++i)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) acc[i] = fmaf(wv[e], th[i * rank + r + e], acc[i]);
+  for (int i = 0; i < ROWS; ++i) acc[i][0] = acc[i][1] = 0.f;
+  const int per = (rank + LR_WAVES - 1) / LR_WAVES, r0 = wid * per, r1 = min(rank, r0 + per);
+#pragma unroll 8
+  for (int r = r0; r < r1; ++r) {
+    float w0 = 0.f, w1 = 0.f;
+    if (both) tm_load2<T>(w + (size_t)r * C + c, w0, w1);
+    else {
+      if (c < C) w0 = to_f(w[(size_t)r * C + c]);
+      if (c + 1 < C) w1 = to_f(w[(size_t)r * C + c + 1]);
     }
-  } else {
-    for (int r = 0; r < rank; ++r) {
-      const float wv = to_f(wc[r]);
 #pragma unroll
-      for (int i = 0; i < LR_ROWS; ++i) acc[i] = fmaf(wv, th[i * rank + r], acc[i]);
+    for (int i = 0; i < ROWS; ++i) {
+      const float t = th[r * ROWS + i];
+      acc[i][0] = fmaf(w0, t, acc[i][0]);
+      acc[i][1] = fmaf(w1, t, acc[i][1]);
     }
   }
-  for (int i = 0; i < n; ++i) z[(size_t)(t0 + i) * C + c] = acc[i];
+  if (wid > 0)
+#pragma unroll
+    for (int i = 0; i < ROWS; ++i) *(float2*)(part + ((size_t)(wid - 1) * ROWS + i) * 128 + 2 * lane) = make_float2(acc[i][0], acc[i][1]);
+  __syncthreads();
+  if (wid > 0) return;
+  for (int v = 0; v < LR_WAVES - 1; ++v)
+#pragma unroll
+    for (int i = 0; i < ROWS; ++i) {
+      const float2 p = *(const float2*)(part + ((size_t)v * ROWS + i) * 128 + 2 * lane);
+      acc[i][0] += p.x; acc[i][1] += p.y;
+    }
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    if (i >= n) break;
+    float* o = z + (size_t)(t0 + i) * C + c;
+    if (both) *(float2*)o = make_float2(acc[i][0], acc[i][1]);
+    else {
+      if (c < C) o[0] = acc[i][0];
+      if (c + 1 < C) o[1] = acc[i][1];
+    }
+  }
 }
 
 extern "C" int ifx_lowrank_tanh(const float* a, int lda, const void* w, int w_dtype, float* z, int T, int rank, int C, void* stream) {
   IFX_REQUIRE(T >= 0 && rank > 0 && C > 0 && lda >= rank, "lowrank_tanh: bad sizes T=%d rank=%d C=%d", T, rank, C);
-  IFX_REQUIRE((size_t)LR_ROWS * rank * sizeof(float) <= 64 * 1024, "lowrank_tanh: a rank of %d does not fit a workgroup's LDS", rank);
+  const int rows = T <= 16 ? 2 : 16;
+  const size_t lds = ((size_t)rows * rank + (size_t)(LR_WAVES - 1) * rows * 128) * sizeof(float);
+  IFX_REQUIRE(lds <= 64 * 1024, "lowrank_tanh: a rank of %d does not fit a workgroup's LDS", rank);
   if (T == 0) return 0;
-  const dim3 grid((T + LR_ROWS - 1) / LR_ROWS, (C + 255) / 256);
-  const size_t lds = (size_t)LR_ROWS * rank * sizeof(float);
+  const dim3 grid((T + rows - 1) / rows, (C + 127) / 128);
   hipStream_t s = (hipStream_t)stream;
-  if (w_dtype == DT_F32) hipLaunchKernelGGL(lowrank_tanh_kernel<float>, grid, dim3(256), lds, s, a, lda, (const float*)w, z, T, rank, C);
-  else if (w_dtype == DT_BF16) hipLaunchKernelGGL(lowrank_tanh_kernel<bf16_t>, grid, dim3(256), lds, s, a, lda, (const bf16_t*)w, z, T, rank, C);
+#define LR(TY, R) hipLaunchKernelGGL((lowrank_tanh_kernel<TY, R>), grid, dim3(LR_WAVES * WAVE), lds, s, a, lda, (const TY*)w, z, T, rank, C)
+  if (w_dtype == DT_F32) { if (rows == 2) LR(float, 2); else LR(float, 16); }
+  else if (w_dtype == DT_BF16) { if (rows == 2) LR(bf16_t, 2); else LR(bf16_t, 16); }
   else IFX_FAIL("lowrank_tanh: unknown dtype %d", w_dtype);
+#undef LR
   IFX_LAUNCH_CHECK();
 }

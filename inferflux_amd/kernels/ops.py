@@ -1620,9 +1620,9 @@ def shifted_mixes(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, state_
 
 
 def lowrank_tanh(a: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    """tanh(a) W^T in float: ``a`` float32 [T, r] (rows may lie further apart), ``w`` [C, r]; float32 [T, C]."""
+    """tanh(a) W in float: ``a`` float32 [T, r] (rows may lie further apart), ``w`` [r, C]; float32 [T, C]."""
     _check(w, "w", (None, None))
-    C, r = w.shape
+    r, C = w.shape
     T = a.shape[0]
     lda = _check_rows(a, "a", T, r, torch.float32)
     z = torch.empty((T, C), dtype=torch.float32, device=w.device)

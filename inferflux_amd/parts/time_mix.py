@@ -74,7 +74,7 @@ class TimeMix(Mixer):
         W = self.width
         self.w_all = ops.prepare_linear(stacked, tile_rows=16)       # r | k | v | g | w1, for few rows: one product over five inputs
         self.w_each = [self.w_all.part(i * W, (i + 1) * W) for i in range(4)] + [self.w_all.part(4 * W, 4 * W + self.decay_rank)]
-        self.w2 = tensors[nm["w2"]].contiguous()
+        self.w2 = tensors[nm["w2"]].t().contiguous()                 # [rank, width]: neighbouring lanes read neighbouring channels
         self.w_o = ops.prepare_linear(tensors[nm["o"]])
         wide = lambda k: tensors[nm[k]].float().contiguous()         # float whatever the file holds
         self.w0, self.u, self.norm_w = wide("w0"), wide("u"), wide("norm")

@@ -199,12 +199,12 @@ def test_mixes_with_the_row_before_over_steps(dtype, H):
 
 
 @pytest.mark.parametrize("wdtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("T,rank,C", [(1, 12, 48), (37, 5, 300), (130, 64, 512), (9, 128, 1024)])
+@pytest.mark.parametrize("T,rank,C", [(1, 12, 48), (37, 5, 300), (130, 64, 512), (9, 128, 1024), (20, 3, 77)])
 def test_the_decays_inner_product(wdtype, T, rank, C):
     a = rnd(1, T, rank + 7, scale=2.0).float()
-    w = rnd(2, C, rank).to(DT[wdtype])
+    w = rnd(2, rank, C).to(DT[wdtype])
     got = ops.lowrank_tanh(a.to(DEV)[:, 7:], w.to(DEV)).cpu()
-    assert rel_err(got, T64(np.tanh(N64(a)[:, 7:]) @ N64(w).T)) < 2e-6
+    assert rel_err(got, T64(np.tanh(N64(a)[:, 7:]) @ N64(w))) < 2e-6
 
 
 def _time_mix_inputs(seed, T, H, d, dt):
