@@ -80,6 +80,7 @@ struct TileArgs {
   float* part_o;          // [T, nH, max_splits, D]
   float* part_ml;         // [T, nH, max_splits, 2]
   const int* order;       // as in attn_mfma.hip's tile kernel
+  const float* sinks;     // [nH]: a score per head that joins its softmax's denominator where the output is written, or null
 };
 
 typedef unsigned int uintx4 __attribute__((ext_vector_type(4)));
@@ -362,7 +363,8 @@ void attn_prefill_kernel(TileArgs a) {
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) *(floatx4*)(po + 16 * dt + 4 * g4) = q[qt].o[dt];
     } else {
-      const float inv = l > 0.f ? 1.f / l : 0.f;
+      const float inv = a.sinks ? finish_factor(q[qt].m * a.scale_log2e, l, 0, 0.f, nullptr, row * a.nH + head, a.sinks, a.nH)
+                                : (l > 0.f ? 1.f / l : 0.f);
       bf16_t* orow = a.out + (row * a.nH + head) * D;
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) {
@@ -381,7 +383,7 @@ extern "C" int ifx_attn_prefill(const void* q, const void* k_cache, const void* 
                                 const int* q_len, const int* kv_len, const int* block_table, int max_blocks,
                                 int nH, int nKV, int d, int page_size, int window, float scale, int chunk, int max_splits,
                                 float* part_o, float* part_ml, const int* rows, int n_rows, const int* row_req,
-                                const int* positions, const int* order, int order_per_xcd, int n_xcd, void* stream) {
+                                const int* positions, const int* order, int order_per_xcd, int n_xcd, const float* sinks, void* stream) {
   IFX_REQUIRE(d == D, "attn_prefill: built for head_dim %d, called with %d", D, d);
   IFX_REQUIRE(n_tiles >= 0 && nH > 0 && nKV > 0 && nH % nKV == 0, "attn_prefill: bad head counts nH=%d nKV=%d", nH, nKV);
   IFX_REQUIRE(page_size >= 16 && (page_size & (page_size - 1)) == 0, "attn_prefill: page_size %d must be a power of two from 16", page_size);
@@ -401,7 +403,7 @@ extern "C" int ifx_attn_prefill(const void* q, const void* k_cache, const void* 
   }
   TileArgs a{(const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, (bf16_t*)out, tile_req, tile_q0, q_start,
              q_len, kv_len, block_table, max_blocks, nH, nKV, page_size, window, scale * 1.4426950408889634f, page_shift,
-             n_tiles, 0, n_xcd, chunk, max_splits, part_o, part_ml, order};
+             n_tiles, 0, n_xcd, chunk, max_splits, part_o, part_ml, order, sinks};
   const long long items = (long long)n_tiles * nH * max_splits;
   IFX_REQUIRE(items <= (1LL << 30), "attn_prefill: too many tiles for one launch");
   IFX_REQUIRE(!order || (order_per_xcd > 0 && (long long)n_xcd * order_per_xcd >= items && order_per_xcd <= items),
@@ -415,6 +417,7 @@ extern "C" int ifx_attn_prefill(const void* q, const void* k_cache, const void* 
     RowArgs m{(const bf16_t*)q, (const bf16_t*)k_cache, (const bf16_t*)v_cache, rows, row_req, positions, block_table,
               part_o, part_ml, (bf16_t*)out, max_blocks, n_rows, nH, nKV, page_size, window, chunk, max_splits,
               scale * 1.4426950408889634f, 1};
+    m.sinks = sinks;
     hipLaunchKernelGGL(attn_rows_merge_kernel, dim3(n_rows, nH), dim3(WAVE * merge_waves(max_splits)), 0, s, m);
   }
   IFX_LAUNCH_CHECK();

@@ -106,8 +106,8 @@ __global__ __launch_bounds__(LR_WAVES * WAVE) void lowrank_tanh_kernel(const flo
   float* part = lr_lds + rank * ROWS;
   const int t0 = blockIdx.x * ROWS, n = min(ROWS, rows - t0), wid = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   for (int x = threadIdx.x; x < ROWS * rank; x += LR_WAVES * WAVE) {
-    const int tt = x / rank, r = x - tt * rank;
-    th[r * ROWS + tt] = tt < n ? tanhf(a[(size_t)(t0 + tt) * lda + r]) : 0.f;
+    const int r = x / ROWS, tt = x % ROWS;
+    th[x] = tt < n ? tanhf(a[(size_t)(t0 + tt) * lda + r]) : 0.f;
   }
   __syncthreads();
   const int c = blockIdx.y * 128 + 2 * lane;          // (C is even where two channels are read at once)
@@ -116,19 +116,30 @@ __global__ __launch_bounds__(LR_WAVES * WAVE) void lowrank_tanh_kernel(const flo
 #pragma unroll
   for (int i = 0; i < ROWS; ++i) acc[i][0] = acc[i][1] = 0.f;
   const int per = (rank + LR_WAVES - 1) / LR_WAVES, r0 = wid * per, r1 = min(rank, r0 + per);
-#pragma unroll 8
-  for (int r = r0; r < r1; ++r) {
-    float w0 = 0.f, w1 = 0.f;
-    if (both) tm_load2<T>(w + (size_t)r * C + c, w0, w1);
-    else {
-      if (c < C) w0 = to_f(w[(size_t)r * C + c]);
-      if (c + 1 < C) w1 = to_f(w[(size_t)r * C + c + 1]);
+  // eight channels' pairs of weights are asked for at once, from places that exist (what they give past the ends is dropped)
+  for (int rb = r0; rb < r1; rb += 8) {
+    float w0[8], w1[8];
+    if (C % 2 == 0) {
+      const T* wc = w + min(c, C - 2);
+#pragma unroll
+      for (int u = 0; u < 8; ++u) tm_load2<T>(wc + (size_t)min(rb + u, rank - 1) * C, w0[u], w1[u]);
+    } else {
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const T* wr = w + (size_t)min(rb + u, rank - 1) * C;
+        w0[u] = to_f(wr[min(c, C - 1)]);
+        w1[u] = to_f(wr[min(c + 1, C - 1)]);
+      }
     }
 #pragma unroll
-    for (int i = 0; i < ROWS; ++i) {
-      const float t = th[r * ROWS + i];
-      acc[i][0] = fmaf(w0, t, acc[i][0]);
-      acc[i][1] = fmaf(w1, t, acc[i][1]);
+    for (int u = 0; u < 8; ++u) {
+      if (rb + u >= r1) break;
+#pragma unroll
+      for (int i = 0; i < ROWS; ++i) {
+        const float t = th[(rb + u) * ROWS + i];
+        acc[i][0] = fmaf(w0[u], t, acc[i][0]);
+        acc[i][1] = fmaf(w1[u], t, acc[i][1]);
+      }
     }
   }
   if (wid > 0)

@@ -234,11 +234,11 @@ def paged_attention(q: torch.Tensor, cache, ctx, window: Optional[int], scale: f
     T, nH, d = q.shape
     table = ctx.block_table(cache.group)
     keep_first = int(keep_first or 0) if window else 0
-    extras = keep_first > 0 or sink is not None or gate is not None or sinks is not None or bool(block)
+    other = keep_first > 0 or sink is not None or gate is not None or bool(block)      # (a sink score per head some kernels do take)
+    extras = other or sinks is not None
     if not ops.mfma_attention_supported(q.dtype, d, cache.page_size) or cache.v.shape[2] != d:
         # values of another width than the keys, or heads wider than a wave's registers hold: one shared kv head (attention
         # through a latent) has a matrix-core kernel of its own, everything else (32-bit, odd sizes) the plain kernel
-        other = keep_first > 0 or sink is not None or gate is not None or bool(block)      # (a sink score per head it does take)
         if not other and ops.wide_attention_supported(q.dtype, cache.k.shape[1], d, cache.v.shape[2], cache.page_size):
             chunk, splits = ops.wide_launch_shape(T, nH, ctx.kv_bound)
             return ops.attention_wide(q, cache.k, cache.v, ctx.row_req, ctx.positions, table, window, scale, chunk, splits, sinks)
@@ -250,7 +250,7 @@ def paged_attention(q: torch.Tensor, cache, ctx, window: Optional[int], scale: f
     qt, splits, chunk = 1, 1, 0
     if tiled.any():
         qt, splits, chunk = choose_tiling(ctx.h_q_len[tiled], ctx.h_kv_len[tiled], nH, lambda t: ops.attention_tile_rows(d, t),
-                                          tall_direct=d == ops.DIRECT_TILE_HEAD_DIM and not extras)
+                                          tall_direct=d == ops.DIRECT_TILE_HEAD_DIM and not other)
     tile_rows = ops.attention_tile_rows(d, qt)
     w = ctx.derived(("attention_work_lists", n_kv, tile_rows, nH, splits, chunk, window, d),
                     lambda: _work_lists(ctx, n_kv, tile_rows, nH, splits, chunk, window, ops.row_waves_fit(nH, n_kv, d, ops.ROW_MAX_WAVES)))

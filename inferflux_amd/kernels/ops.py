@@ -2049,7 +2049,7 @@ def attention_tiles(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
 
     ``order`` (int32 [8 * n], from ``attention.tile_order``) says which work item each workgroup of the launch
     takes; every item must appear exactly once (-1: a workgroup without work).  The result does not depend on it."""
-    extras = bool(keep_first) or sink is not None or gate is not None or sinks is not None or bool(block)      # (the kernel that loads straight into LDS has none of them)
+    extras = bool(keep_first) or sink is not None or gate is not None or bool(block)      # (the kernel that loads straight into LDS has none of them; it does take sinks per head)
     T, nH, d, nKV, page_size, mod = _attn_common(q, k_cache, v_cache, qt, not extras)
     _, _, entry, rows_fn = _tile_module(d, qt, not extras)
     if mod.fn(rows_fn, ())() != attention_tile_rows(d, qt):
@@ -2089,7 +2089,9 @@ def attention_tiles(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     if entry == "ifx_attn_tiles":
         _call(mod, entry, types + (I, I, F, P, P, I, P), *args, *_attn_extras(T, nH, keep_first, sink, gate, sinks, block), _stream())
     else:
-        _call(mod, entry, types + (P,), *args, _stream())
+        if sinks is not None:
+            _check(sinks, "sinks", (nH,), torch.float32)
+        _call(mod, entry, types + (P, P), *args, _ptr(sinks), _stream())
 
 
 # ----------------------------------------------------------------------------------------

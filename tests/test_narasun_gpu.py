@@ -150,6 +150,35 @@ def test_a_sink_per_head_joins_the_denominator(dtype, n, nH, nKV, d, dv):
     assert rel_err(without, T64(want)) > 0.05
 
 
+@pytest.mark.parametrize("d,qt", [(128, 2), (128, 1), (64, 2), (32, 1)])
+@pytest.mark.parametrize("past,splits", [(0, 1), (0, 3), (130, 1), (130, 4)])
+def test_sinks_in_the_tile_kernels(d, qt, past, splits):
+    """A prompt's portion behind ``past`` keys through the kernels for tiles of rows (at head size 128 the tall tiles are the
+    kernel that loads straight into LDS), whole and with the keys cut into splits; sinks from far below every score to above
+    it, and rows whose one large score is for a key in the first split."""
+    n, nH, nKV, P = 300, 4, 2, 16
+    total = past + n
+    q, k, v = rnd(1, n, nH, d).bfloat16().double(), rnd(2, total, nKV, d).bfloat16().double(), rnd(3, total, nKV, d).bfloat16().double()
+    scale, sinks = d ** -0.5, torch.tensor([3.0, -40.0, 0.0, 12.0])
+    for i in range(0, n, 7):
+        q[i] = (4.0 * k[i % 11].repeat_interleave(nH // nKV, 0)).bfloat16().double()
+    K, V, table = _paged(k, v, torch.bfloat16)
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=DEV)
+    rows = ops.attention_tile_rows(d, qt)
+    q0 = list(range(0, n, rows))
+    chunk = -(-(-(-total // splits)) // 64) * 64 if splits > 1 else 0
+    out = torch.zeros(n, nH * d, dtype=torch.bfloat16, device=DEV)
+    ops.attention_tiles(q.bfloat16().to(DEV), K, V, out, i32([0] * len(q0)), i32(q0), i32([0]), i32([n]), i32([total]), table, None, scale, qt, chunk,
+                        splits, torch.arange(n, dtype=torch.int32, device=DEV), i32([0] * n), torch.arange(past, total, dtype=torch.int32, device=DEV),
+                        sinks=sinks.to(DEV))
+    full = np.concatenate([np.zeros((past, nH, d)), N64(q)])
+    want = np.stack([pn.causal_softmax(full[:, h] @ N64(k[:, h // 2]).T * scale, float(sinks[h])) @ N64(v[:, h // 2]) for h in range(nH)], axis=1)
+    want = want[past:].reshape(n, nH * d)
+    assert rel_err(out.cpu(), T64(want)) < 2e-2
+    heads = (out.cpu().double() - T64(want)).reshape(n, nH, d).abs().amax(dim=(0, 2)) / T64(want).reshape(n, nH, d).abs().amax(dim=(0, 2))
+    assert float(heads.max()) < 3e-2        # (a head whose sink takes nearly everything has small outputs of its own)
+
+
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("T,nH,nKV,d,dv", [(5, 4, 2, 16, 24), (200, 4, 2, 64, 64), (150, 3, 1, 10, 14), (130, 2, 2, 32, 16)])
 def test_query_temperature_multiplies_the_queries_alone(dtype, T, nH, nKV, d, dv):
