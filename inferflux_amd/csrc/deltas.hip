@@ -120,6 +120,31 @@ __global__ __launch_bounds__(256) void add_terms_rmsnorm_kernel(float* __restric
   }
 }
 
+template <typename TO, int NV>
+__global__ __launch_bounds__(256) void join_stream4_kernel(const float* __restrict__ stream, Pieces pieces, const float* __restrict__ other,
+                                                           TO* __restrict__ out, int H) {
+  const size_t t = blockIdx.x;
+  float x[NV][4], y[NV][4];
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int i = 4 * (threadIdx.x + 256 * v);
+    if (i < H) {
+      dl_load4(stream, DT_F32, t * H + i, x[v]);
+      dl_load4(other, DT_F32, t * H + i, y[v]);
+    }
+  }
+  add_pieces4<NV>(pieces, t, H, x);
+#pragma unroll
+  for (int v = 0; v < NV; ++v) {
+    const int i = 4 * (threadIdx.x + 256 * v);
+    if (i < H) {
+      dl_store4(out + t * 2 * H + i, x[v]);
+      dl_store4(out + t * 2 * H + H + i, y[v]);
+    }
+  }
+}
+
+// any width
 template <typename TO>
 __global__ __launch_bounds__(256) void join_stream_kernel(const float* __restrict__ stream, Pieces pieces, const float* __restrict__ other,
                                                           TO* __restrict__ out, int H) {
@@ -185,6 +210,21 @@ extern "C" int ifx_join_stream(const float* x, int n_terms, const void* const* p
   if (T == 0) return 0;
   const dim3 grid(T, (2 * H + 255) / 256);
   hipStream_t s = (hipStream_t)stream;
+  if (H % 4 == 0 && H <= 8192 && (out_dtype == DT_F32 || out_dtype == DT_BF16)) {
+#define JOIN(TO, NV) hipLaunchKernelGGL((join_stream4_kernel<TO, NV>), dim3(T), dim3(256), 0, s, x, pieces, other, (TO*)out, H)
+#define JOIN_ALL(TO)                 \
+  do {                               \
+    if (H <= 1024) JOIN(TO, 1);      \
+    else if (H <= 2048) JOIN(TO, 2); \
+    else if (H <= 4096) JOIN(TO, 4); \
+    else JOIN(TO, 8);                \
+  } while (0)
+    if (out_dtype == DT_F32) JOIN_ALL(float);
+    else JOIN_ALL(bf16_t);
+#undef JOIN_ALL
+#undef JOIN
+    IFX_LAUNCH_CHECK();
+  }
   if (out_dtype == DT_F32) hipLaunchKernelGGL(join_stream_kernel<float>, grid, dim3(256), 0, s, x, pieces, other, (float*)out, H);
   else if (out_dtype == DT_BF16) hipLaunchKernelGGL(join_stream_kernel<bf16_t>, grid, dim3(256), 0, s, x, pieces, other, (bf16_t*)out, H);
   else IFX_FAIL("join_stream: unknown out dtype %d", out_dtype);

@@ -167,15 +167,15 @@ __global__ __launch_bounds__(LR_WAVES * WAVE) void lowrank_tanh_kernel(const flo
 
 extern "C" int ifx_lowrank_tanh(const float* a, int lda, const void* w, int w_dtype, float* z, int T, int rank, int C, void* stream) {
   IFX_REQUIRE(T >= 0 && rank > 0 && C > 0 && lda >= rank, "lowrank_tanh: bad sizes T=%d rank=%d C=%d", T, rank, C);
-  const int rows = T <= 16 ? 2 : 16;
+  const int rows = T <= 16 ? 2 : (T <= 128 ? 4 : 16);         // (few rows: more workgroups)
   const size_t lds = ((size_t)rows * rank + (size_t)(LR_WAVES - 1) * rows * 128) * sizeof(float);
   IFX_REQUIRE(lds <= 64 * 1024, "lowrank_tanh: a rank of %d does not fit a workgroup's LDS", rank);
   if (T == 0) return 0;
   const dim3 grid((T + rows - 1) / rows, (C + 127) / 128);
   hipStream_t s = (hipStream_t)stream;
 #define LR(TY, R) hipLaunchKernelGGL((lowrank_tanh_kernel<TY, R>), grid, dim3(LR_WAVES * WAVE), lds, s, a, lda, (const TY*)w, z, T, rank, C)
-  if (w_dtype == DT_F32) { if (rows == 2) LR(float, 2); else LR(float, 16); }
-  else if (w_dtype == DT_BF16) { if (rows == 2) LR(bf16_t, 2); else LR(bf16_t, 16); }
+  if (w_dtype == DT_F32) { if (rows == 2) LR(float, 2); else if (rows == 4) LR(float, 4); else LR(float, 16); }
+  else if (w_dtype == DT_BF16) { if (rows == 2) LR(bf16_t, 2); else if (rows == 4) LR(bf16_t, 4); else LR(bf16_t, 16); }
   else IFX_FAIL("lowrank_tanh: unknown dtype %d", w_dtype);
 #undef LR
   IFX_LAUNCH_CHECK();
