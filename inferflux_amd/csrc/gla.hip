@@ -216,6 +216,7 @@ struct CombineArgs {
   int H, d, dv, parts, dp;
 };
 
+#define WALK_AHEAD 8
 __global__ __launch_bounds__(256) void gla_combine_kernel(CombineArgs a) {
   const size_t per = (size_t)a.H * a.dv * a.parts * a.dp;
   const size_t e = (size_t)blockIdx.x * 256 + threadIdx.x;
@@ -228,11 +229,20 @@ __global__ __launch_bounds__(256) void gla_combine_kernel(CombineArgs a) {
   float* slot = a.state + (size_t)a.slots[r] * a.state_stride + a.state_offset + e;
   if (i >= a.d) return;                   // (padding: zero for ever)
   float S = *slot;
-  for (int c = c0; c < c1; ++c) {
-    float* cs = a.chunk_state + (size_t)c * per + e;
-    const float mine = *cs;
-    *cs = S;
-    S = fmaf(expf(a.chunk_loga[(size_t)c * a.H * a.d + head * a.d + i]), S, mine);
+  for (int k0 = c0; k0 < c1; k0 += WALK_AHEAD) {        // (the loads of several chunks are on their way at once)
+    float mine[WALK_AHEAD], keep[WALK_AHEAD];
+#pragma unroll
+    for (int u = 0; u < WALK_AHEAD; ++u) {
+      const int c = min(k0 + u, c1 - 1);
+      mine[u] = a.chunk_state[(size_t)c * per + e];
+      keep[u] = a.chunk_loga[(size_t)c * a.H * a.d + head * a.d + i];
+    }
+#pragma unroll
+    for (int u = 0; u < WALK_AHEAD; ++u) {
+      if (k0 + u >= c1) break;
+      a.chunk_state[(size_t)(k0 + u) * per + e] = S;
+      S = fmaf(expf(keep[u]), S, mine[u]);
+    }
   }
   *slot = S;
 }
