@@ -174,21 +174,11 @@ def compile_module(name: str, variant: Variant = (), force: bool = False) -> str
             label = f"{name}{_variant_tag(variant)}"
             _progress(f"compiling {label} for {'the host' if host else ARCH} ...")
             t0 = time.time()
-            proc = subprocess.Popen(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True, cwd=out_dir)
-            done = threading.Event()
-
-            def tick():
-                while not done.wait(20.0):
-                    _progress(f"still compiling {label} ({time.time() - t0:.0f} s)")
-
-            th = threading.Thread(target=tick, daemon=True)
-            th.start()
-            log, _ = proc.communicate()
-            done.set()
+            proc = subprocess.run(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True, cwd=out_dir)
             if proc.returncode != 0 or not os.path.isfile(tmp):
                 if os.path.exists(tmp):
                     os.unlink(tmp)
-                raise KernelBuildError(f"{os.path.basename(cmd[0])} failed for {label} (exit {proc.returncode}):\n{' '.join(cmd)}\n{log}")
+                raise KernelBuildError(f"{os.path.basename(cmd[0])} failed for {label} (exit {proc.returncode}):\n{' '.join(cmd)}\n{proc.stdout}")
             os.replace(tmp, out)
             # Drop libraries of the same module built from older sources.
             prefix = f"{_stem(name, variant)}."
